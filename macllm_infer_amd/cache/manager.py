@@ -15,7 +15,7 @@ step; ``finish`` gives everything back (:1840-1852).
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Dict, Hashable, List, Optional, Sequence, Tuple
 
 import numpy as np
@@ -30,17 +30,42 @@ class KVNeed:
     """Token-proportional cache: per token, keys of ``num_kv_heads`` x ``head_dim`` and values of
     ``num_kv_heads`` x ``value_dim`` (None: the keys' width); ``window`` = how many of the most recent
     tokens must stay (None = all); ``keep_first`` = how many of a request's first tokens stay as well, however
-    far the window has moved on."""
+    far the window has moved on; ``chunk`` (in place of a window) = the tokens of a request's current chunk of that many
+    positions, counted from its start, must stay."""
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     value_dim: Optional[int] = None
     keep_first: int = 0
+    chunk: Optional[int] = None
     token_proportional = True             # what tells this need from one of fixed size, whatever its class
 
     @property
     def value_width(self) -> int:
         return self.head_dim if self.value_dim is None else self.value_dim
+
+    @property
+    def keeps_every_key(self) -> bool:
+        return self.window is None and self.chunk is None
+
+    @property
+    def span(self) -> int:
+        """What the host-side core takes: a window's size, the negated size of chunks, or 0 for every key."""
+        return -self.chunk if self.chunk else self.window or 0
+
+    def same_rows(self, other: "KVNeed") -> bool:
+        return ((self.num_kv_heads, self.head_dim, self.value_width)
+                == (other.num_kv_heads, other.head_dim, other.value_width))
+
+    def covering(self, other: "KVNeed") -> "KVNeed":
+        """This need, keeping as well what ``other``, which reads the same rows, still sees."""
+        if (self.window, self.keep_first, self.chunk) == (other.window, other.keep_first, other.chunk):
+            return self
+        if self.keeps_every_key or other.keeps_every_key:
+            return replace(self, window=None, keep_first=0, chunk=None)
+        # a chunk of c positions never reaches further back than a window of c keys
+        most = max(self.window or self.chunk, other.window or other.chunk)
+        return replace(self, window=most, keep_first=max(self.keep_first, other.keep_first), chunk=None)
 
 
 @dataclass(frozen=True)
@@ -66,11 +91,11 @@ class Core:
     """The host-side core of one cache manager (``csrc/hostcore.cpp``): every group's page pool
     and block tables, the slot pool and the requests' lengths."""
 
-    def __init__(self, page_sizes: Sequence[int], num_pages: Sequence[int], windows: Sequence[Optional[int]],
+    def __init__(self, page_sizes: Sequence[int], num_pages: Sequence[int], spans: Sequence[int],
                  max_requests: int, kept_first: Optional[Sequence[int]] = None):
         self.lib = native.lib()
         sizes, pages = native.as_ints(list(page_sizes)), native.as_ints(list(num_pages))
-        spans = native.as_ints([window or -1 for window in windows])
+        spans = native.as_ints(list(spans))
         self.pointer = self.lib.hc_create(len(sizes), native.int_pointer(sizes), native.int_pointer(pages),
                                           native.int_pointer(spans), max_requests)
         if not self.pointer:
@@ -173,6 +198,13 @@ class CacheManager:
         self.max_requests = max_requests
         self.requests: Dict[Hashable, RequestCache] = {}
         self._state_tensors: List[torch.Tensor] = []
+        # a mixer whose rows others read keeps what any of them still sees
+        needs = {key: list(key_needs) for key, key_needs in needs.items()}
+        for reader, source in shared_kv.items():
+            mine = [need for need in needs[reader] if getattr(need, "token_proportional", False)]
+            for index, need in enumerate(needs[source]):
+                if getattr(need, "token_proportional", False) and mine and need.same_rows(mine[0]):
+                    needs[source][index] = need.covering(mine[0])
         group_of: Dict[KVNeed, int] = {}
         layer_of: Dict[Hashable, Tuple[int, int]] = {}
         for key, key_needs in needs.items():
@@ -197,7 +229,7 @@ class CacheManager:
                     raise TypeError(f"unknown cache need {need!r}")
             self.entries[key] = entry
         self.core = Core([group.page_size for group in self.groups], [group.num_pages for group in self.groups],
-                         [group.need.window for group in self.groups], max_requests,
+                         [group.need.span for group in self.groups], max_requests,
                          [getattr(group.need, "keep_first", 0) for group in self.groups])
         self.slots = SlotPool.view(self.core.lib.hc_slot_pool(self.core.pointer), self.core)
         for index, group in enumerate(self.groups):
@@ -209,7 +241,7 @@ class CacheManager:
                 if key in shared_kv:
                     own = [need for need in needs[key] if getattr(need, "token_proportional", False)]
                     theirs = self.groups[layer_of[source][0]].need
-                    if not own or own[0] != theirs:
+                    if not own or not own[0].same_rows(theirs):
                         raise ValueError(f"{key} cannot read the cache of {source}: their needs differ")
                 group, layer = layer_of[source]
                 entry.group = group
@@ -295,7 +327,7 @@ class CacheManager:
 
     def stats(self) -> dict:
         return {
-            "groups": [{"window": group.need.window, "layers": len(group.members),
+            "groups": [{"window": group.need.window, "chunk": group.need.chunk, "layers": len(group.members),
                         "total_pages": group.num_pages, "free_pages": group.pool.free_count,
                         "used_pages": group.pool.used_count} for group in self.groups],
             "total_slots": self.max_requests, "free_slots": self.slots.free_count,

@@ -1,7 +1,7 @@
 from .spec import (SILU_GLU, AttentionSpec, ClampedGLUSpec, ConfigError, GatedLinearAttentionSpec, GeneralDeltaSpec, HashedBigramSpec,
                    InterleavedRopeSpec,
-                   LatentAttentionSpec, LayerNormSpec, LayerSpec, LightningAttentionSpec, LogDistanceBiasSpec, Mamba2Spec, MixerSlot,
-                   ModelSpec, NoPositionSpec, PolyNormFFNSpec, PowerReluSpec, RampScalingSpec, RetentionSpec, RmsNormSpec, RopeSpec,
+                   LatentAttentionSpec, LayerNormSpec, LayerSpec, LightningAttentionSpec, LinearDistanceBiasSpec, LogDistanceBiasSpec, Mamba2Spec,
+                   MixerSlot, ModelSpec, NoPositionSpec, PolyNormFFNSpec, PowerReluSpec, RampScalingSpec, RetentionSpec, RmsNormSpec, RopeSpec,
                    RoutedExpertsSpec, ScheduleEntry, StreamInjection, SwiGLUSpec, TanhNormSpec, WavelengthScalingSpec)
 from .registry import (config_from_dict, load_config, register_architecture,
                        registered_architectures)
@@ -11,6 +11,7 @@ from .lutosun import LutosunConfig
 from .motolix import MotolixConfig
 from .pemarax import PemaraxConfig
 from .pipizen import PipizenConfig
+from .sazavik import SazavikConfig
 
 register_architecture(FalconH1Config)
 register_architecture(MukutarConfig)
@@ -18,9 +19,10 @@ register_architecture(LutosunConfig)
 register_architecture(MotolixConfig)
 register_architecture(PemaraxConfig)
 register_architecture(PipizenConfig)
+register_architecture(SazavikConfig)
 
 __all__ = ["AttentionSpec", "ClampedGLUSpec", "ConfigError", "FalconH1Config", "GatedLinearAttentionSpec", "GeneralDeltaSpec", "HashedBigramSpec",
-           "InterleavedRopeSpec", "LatentAttentionSpec", "LayerNormSpec", "LayerSpec", "LightningAttentionSpec", "LogDistanceBiasSpec", "LutosunConfig",
+           "InterleavedRopeSpec", "LatentAttentionSpec", "LayerNormSpec", "LayerSpec", "LightningAttentionSpec", "LinearDistanceBiasSpec", "LogDistanceBiasSpec", "LutosunConfig",
            "Mamba2Spec", "MixerSlot", "ModelSpec", "MotolixConfig", "MukutarConfig", "NoPositionSpec", "PemaraxConfig", "PipizenConfig", "PolyNormFFNSpec", "PowerReluSpec", "RampScalingSpec", "RetentionSpec",
-           "RmsNormSpec", "RopeSpec", "RoutedExpertsSpec", "SILU_GLU", "ScheduleEntry", "StreamInjection", "SwiGLUSpec", "TanhNormSpec", "WavelengthScalingSpec",
+           "RmsNormSpec", "RopeSpec", "RoutedExpertsSpec", "SILU_GLU", "SazavikConfig", "ScheduleEntry", "StreamInjection", "SwiGLUSpec", "TanhNormSpec", "WavelengthScalingSpec",
            "config_from_dict", "load_config", "register_architecture", "registered_architectures"]

@@ -155,6 +155,23 @@ class LogDistanceBiasSpec:
 
 
 @dataclass(frozen=True)
+class LinearDistanceBiasSpec:
+    """No rotation; the score of a key at distance n behind the query loses slope_h * n, with the fixed slopes
+    slope_h = 2^(-``exponent`` (h + 1) / ``num_heads``) of the query heads h = 0, 1, ..."""
+    num_heads: int
+    exponent: float = 8.0
+    kind: str = "linear_distance"
+
+    def validate(self, head_dim: int) -> None:
+        _require(self.num_heads > 0, "a distance bias needs the number of query heads")
+        _require(0 < self.exponent < 1000, "the distance bias's exponent must be positive")
+
+    @property
+    def slopes(self) -> Tuple[float, ...]:
+        return tuple(2.0 ** (-self.exponent * (head + 1) / self.num_heads) for head in range(self.num_heads))
+
+
+@dataclass(frozen=True)
 class AttentionSpec:
     """Grouped-query causal attention (src/architecture.rs:139-151).
 
@@ -208,6 +225,17 @@ class AttentionSpec:
     head_norm: Optional[str] = None
     head_norm_weight: bool = False
     head_norm_eps: float = 1e-6
+    # in place of a window: the sequence is cut into chunks of this many positions, counted from its start, and a query
+    # sees the keys of its own chunk up to its own
+    chunk: Optional[int] = None
+    # the concatenated heads are multiplied by sigmoid(W_g x), element by element, before the output projection
+    # (tensor ``g_proj`` beside the q, k and v projections, no bias)
+    out_gate: bool = False
+    # (coef, every): a query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1)
+    query_temperature: Optional[Tuple[float, int]] = None
+    # False: the mixer has no k and v projections (nor a k norm) and writes no cache; it attends to the keys and values
+    # that another mixer cached (the schedule entry's ``kv_from``)
+    own_rows: bool = True
     kind: str = "attention"
 
     @property
@@ -221,7 +249,7 @@ class AttentionSpec:
         _require(self.num_heads % self.num_kv_heads == 0,
                  f"num_attention_heads {self.num_heads} is not a multiple of "
                  f"num_key_value_heads {self.num_kv_heads}")
-        _require(self.head_dim > 0 and self.head_dim % 2 == 0,
+        _require(self.head_dim > 0 and (self.head_dim % 2 == 0 or self.head_norm is not None),
                  f"head_dim {self.head_dim} must be positive and even")
         _require(self.scale > 0, "attention scale must be positive")
         _require(self.window is None or self.window > 0, "attention window must be positive")
@@ -243,6 +271,14 @@ class AttentionSpec:
         _require(self.head_norm is None or self.projection_norm_eps is None,
                  "q and k are normed head by head or as whole projections, not both")
         _require(self.head_norm is None or self.head_norm_eps > 0, "the heads' norm eps must be positive")
+        _require(self.chunk is None or (self.chunk > 0 and self.window is None),
+                 "attention chunks must be positive, and stand in place of a window")
+        _require(not self.out_gate or self.value_rotation_theta is None, "a gate on outputs that are turned back is not known")
+        _require(self.query_temperature is None or self.query_temperature[1] > 0,
+                 "the step of the queries' temperature must be positive")
+        _require(self.own_rows or (not self.values_from_keys and self.projection_norm_eps is None and self.conv_kernel == 0
+                                   and self.value_rotation_theta is None),
+                 "a mixer that reads another's keys has no values from keys, convolution, turned values or whole projections' norm")
         self.position.validate(self.head_dim)
 
 
@@ -327,7 +363,10 @@ class RoutedExpertsSpec:
     (+ ``weight_eps``), times ``route_scale``.  ``routing`` "top_then_softmax": the ``top_k`` largest logits
     z = W_router x + bias (tensor ``router.bias``) are chosen and weighted by the softmax over the chosen logits
     alone, times ``route_scale``.
-    ``renormalize`` False (softmax_then_top): the weights are the chosen s themselves, times ``route_scale``.
+    ``routing`` "sigmoid_then_top": as the first, with s = sigmoid(W_router x) output by output.
+    ``renormalize`` False (with one of the scores s): the weights are the chosen s themselves, times ``route_scale``.
+    ``corrected`` False: the choice is by s alone (no tensor ``correction``).  ``input_weighted``: a weight multiplies its
+    expert's input in place of its output: the sum of expert(w * x).
     ``identity_experts``: the router's last outputs stand for experts whose output is their input; they have no
     matrices, and take part in softmax, correction and choice like the others.  ``groups``: all the router's outputs
     form that many equal groups of neighbours; a group's score is its largest s + correction, and only outputs of the
@@ -347,6 +386,8 @@ class RoutedExpertsSpec:
     groups: int = 0
     kept_groups: int = 0
     shared_gated: bool = True
+    corrected: bool = True
+    input_weighted: bool = False
     kind: str = "routed_experts"
 
     @property
@@ -358,8 +399,10 @@ class RoutedExpertsSpec:
         _require(self.identity_experts >= 0, "the number of identity experts cannot be negative")
         _require(0 < self.top_k <= self.router_outputs,
                  f"a token uses {self.top_k} experts of {self.router_outputs}")
-        _require(self.routing == "softmax_then_top" or (self.renormalize and self.groups == 0 and self.identity_experts == 0),
-                 "groups, identity experts and weights as they are come with the softmax over all experts")
+        _require(self.routing != "top_then_softmax" or (self.renormalize and self.groups == 0 and self.identity_experts == 0
+                                                        and self.corrected),
+                 "groups, identity experts and weights as they are come with scores of all experts")
+        _require(not self.input_weighted or self.identity_experts == 0, "weights on the experts' inputs and identity experts")
         if self.groups:
             _require(self.groups > 0 and self.router_outputs % self.groups == 0,
                      f"{self.router_outputs} experts do not form {self.groups} equal groups")
@@ -367,7 +410,8 @@ class RoutedExpertsSpec:
             _require(self.kept_groups * (self.router_outputs // self.groups) >= self.top_k,
                      f"{self.kept_groups} groups of {self.router_outputs // self.groups} experts hold fewer than the "
                      f"{self.top_k} a token uses")
-        _require(self.routing in ("softmax_then_top", "top_then_softmax"), f"routing {self.routing!r} is not known")
+        _require(self.routing in ("softmax_then_top", "top_then_softmax", "sigmoid_then_top"),
+                 f"routing {self.routing!r} is not known")
         self.activation.validate()
         if self.shared_size is not None:
             _require(self.shared_size > 0 and self.shared_activation is not None,
@@ -558,17 +602,22 @@ class PolyNormFFNSpec:
 @dataclass(frozen=True)
 class SwiGLUSpec:
     """down(act(gate(x) * gate_multiplier) * up(x)) * down_multiplier (src/decoder.rs:261-306), act = SiLU or,
-    with ``activation`` "gelu_tanh", 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))."""
+    with ``activation`` "gelu_tanh", 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))).  Activation "clamped" (``clamp``):
+    the clamped gated activation of gate(x) and up(x) (``ClampedGLUSpec``)."""
     intermediate_size: int
     bias: bool = False
     gate_multiplier: float = 1.0
     down_multiplier: float = 1.0
     activation: str = "silu"
+    clamp: Optional[ClampedGLUSpec] = None
     kind: str = "swiglu"
 
     def validate(self) -> None:
         _require(self.intermediate_size > 0, "intermediate_size must be positive")
-        _require(self.activation in ("silu", "gelu_tanh"), f"the gate's activation {self.activation!r} is not known")
+        _require(self.activation in ("silu", "gelu_tanh", "clamped"), f"the gate's activation {self.activation!r} is not known")
+        _require((self.activation == "clamped") == (self.clamp is not None), "the clamped activation and its numbers come together")
+        if self.clamp is not None:
+            self.clamp.validate()
 
 
 @dataclass(frozen=True)
@@ -649,6 +698,9 @@ class ModelSpec:
     injected_vectors: Tuple[Tuple[str, int], ...] = ()
     # tensors [hidden, 2 hidden] that schedule entries name (``StreamInjection.mix_name``)
     injected_mixes: Tuple[str, ...] = ()
+    # an RMS norm of the embedding output: the stream starts as its rows (None: as the embedding's own)
+    embedding_norm: Optional[RmsNormSpec] = None
+    embedding_norm_name: str = "embed.norm"
     embedding_name: str = "model.embed_tokens"
     final_norm_name: str = "model.norm"
     lm_head_name: str = "lm_head"
@@ -681,6 +733,10 @@ class ModelSpec:
         _require(self.logit_softcap is None or (0 < self.logit_softcap < float("inf")),
                  f"the cap on the logits must be finite and positive, got {self.logit_softcap}")
         self.final_norm.validate()
+        if self.embedding_norm is not None:
+            _require(self.embedding_norm.kind == "rmsnorm" and self.bigram is None,
+                     "the norm of the embedding output is an RMS norm, of one embedding")
+            self.embedding_norm.validate()
         if self.bigram is not None:
             self.bigram.validate()
         vectors = dict(self.injected_vectors)

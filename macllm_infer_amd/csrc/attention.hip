@@ -126,9 +126,11 @@ extern "C" int mi_rope_kv_store(void* qkv, int dtype, long ld, int T, int Hq, in
 //   * q and k are turned by the token's position over the first rotary_dim dims, angle = (float)position *
 //     inv_freq[j], pairs (j, j + rotary_dim / 2) or, interleaved, (2j, 2j + 1); cosines and sines times turn_scale;
 //     q is written back in place, k goes to the token's cache cell;
+//   * with temp_every > 0 the queries are multiplied by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1);
 //   * the values are the v heads of the row or, with values_from_keys, the k heads as they were projected (before
 //     norm and rotation; dv = dh); with value_inv_freq they are turned by the position over all dv dims (half-split
 //     pairs, angle = (float)position * value_inv_freq[m]); they go to the token's transposed cache cell.
+// A row of queries alone (Hkv = 0, no slot_mapping) is one whose keys and values another layer has cached.
 template <typename T>
 __global__ void __launch_bounds__(256)
 attention_prepare_kernel(T* __restrict__ qkv, long ld, int Hq, int Hkv, int dh, int dv, int values_from_keys,
@@ -136,7 +138,7 @@ attention_prepare_kernel(T* __restrict__ qkv, long ld, int Hq, int Hkv, int dh, 
                          int interleaved, float turn_scale,
                          const float* __restrict__ q_norm, const float* __restrict__ k_norm, float norm_eps,
                          int head_norm, const float* __restrict__ q_head_weight, const float* __restrict__ k_head_weight,
-                         float head_eps,
+                         float head_eps, float temp_coef, int temp_every,
                          const float* __restrict__ value_inv_freq, const int* __restrict__ slot_mapping,
                          T* __restrict__ k_base, T* __restrict__ v_base, long page_stride, int page_size) {
   extern __shared__ float prepared_row[];
@@ -215,6 +217,7 @@ attention_prepare_kernel(T* __restrict__ qkv, long ld, int Hq, int Hkv, int dh, 
     __syncthreads();
   }
   if (head_norm == 2) norm_heads();
+  const float temperature = temp_every > 0 ? 1.0f + temp_coef * logf((float)((positions[token] + 1) / temp_every + 1)) : 1.0f;
   long cell = -1, page = 0;
   int offset = 0;
   if (slot_mapping) {
@@ -226,7 +229,7 @@ attention_prepare_kernel(T* __restrict__ qkv, long ld, int Hq, int Hkv, int dh, 
     const int head = item / dh;
     const int j = item - head * dh;
     const float value = prepared_row[item];
-    if (head < Hq) row[item] = from_float<T>(value);
+    if (head < Hq) row[item] = from_float<T>(value * temperature);
     else if (cell >= 0)
       k_base[page * page_stride + ((long)(head - Hq) * page_size + offset) * dh + j] = from_float<T>(value);
   }
@@ -252,9 +255,10 @@ extern "C" int mi_attention_prepare(void* qkv, int dtype, long ld, int T, int Hq
                                     int interleaved, float turn_scale,
                                     const float* q_norm, const float* k_norm, float norm_eps,
                                     int head_norm, const float* q_head_weight, const float* k_head_weight, float head_eps,
-                                    const float* value_inv_freq, const int* slot_mapping, void* k_base, void* v_base,
+                                    float temp_coef, int temp_every, const float* value_inv_freq, const int* slot_mapping, void* k_base, void* v_base,
                                     long page_stride, int page_size, hipStream_t stream) {
-  if (!qkv || !positions || T <= 0 || Hq <= 0 || Hkv <= 0 || dh <= 0 || dv <= 0) return ERR_BAD_ARGUMENT;
+  if (!qkv || !positions || T <= 0 || Hq <= 0 || Hkv < 0 || dh <= 0 || dv <= 0 || temp_every < 0) return ERR_BAD_ARGUMENT;
+  if (Hkv == 0 && (slot_mapping || q_norm || values_from_keys)) return ERR_BAD_ARGUMENT;      // queries alone
   if (rotary_dim < 0 || rotary_dim > dh || (rotary_dim & 1) || (rotary_dim > 0 && !inv_freq)) return ERR_BAD_ARGUMENT;
   if (values_from_keys && dv != dh) return ERR_BAD_ARGUMENT;
   if (value_inv_freq && (dv & 1)) return ERR_BAD_ARGUMENT;
@@ -271,13 +275,13 @@ extern "C" int mi_attention_prepare(void* qkv, int dtype, long ld, int T, int Hq
     attention_prepare_kernel<float><<<T, 256, lds, stream>>>((float*)qkv, ld, Hq, Hkv, dh, dv, values_from_keys, positions,
                                                              inv_freq, rotary_dim, interleaved, turn_scale, q_norm, k_norm,
                                                              norm_eps, head_norm, q_head_weight, k_head_weight, head_eps,
-                                                             value_inv_freq, slot_mapping, (float*)k_base, (float*)v_base,
+                                                             temp_coef, temp_every, value_inv_freq, slot_mapping, (float*)k_base, (float*)v_base,
                                                              page_stride, page_size);
   else if (dtype == DT_BF16)
     attention_prepare_kernel<bf16_t><<<T, 256, lds, stream>>>((bf16_t*)qkv, ld, Hq, Hkv, dh, dv, values_from_keys,
                                                               positions, inv_freq, rotary_dim, interleaved, turn_scale,
                                                               q_norm, k_norm, norm_eps, head_norm, q_head_weight,
-                                                              k_head_weight, head_eps, value_inv_freq, slot_mapping,
+                                                              k_head_weight, head_eps, temp_coef, temp_every, value_inv_freq, slot_mapping,
                                                               (bf16_t*)k_base, (bf16_t*)v_base, page_stride, page_size);
   else
     return ERR_BAD_ARGUMENT;
@@ -289,7 +293,8 @@ extern "C" int mi_attention_prepare(void* qkv, int dtype, long ld, int T, int Hq
 // Works for any head_dim <= 256, any page size, any group size, float32 and bfloat16; the float32 path of
 // the whole model uses it for prompts and for decoding alike.
 //   s = q.k * scale;  visible keys: position <= query position, and
-//   query - key < window when window > 0 (reference: src/decoder.rs:4515-4532); with kept > 0 the keys at
+//   query - key < window when window > 0 (reference: src/decoder.rs:4515-4532), or of the query's own chunk of
+//   -window positions when window < 0 (first_visible_key); with kept > 0 the keys at
 //   positions below kept stay visible behind the window (the first tokens of a sequence, at their true positions);
 //   softmax in float32 (reference: src/decoder.rs:4665-4667).
 // `slopes` (optional, float32 per query head): a position encoding that is a bias on the scores,
@@ -336,8 +341,7 @@ paged_attention_kernel(const T* __restrict__ q, long q_ld, int Hq, int Hkv, int 
   const int head = blockIdx.y;
   const int run = blockIdx.z;
   const int query_position = positions[token];
-  int first_key = 0;
-  if (window > 0 && query_position - window + 1 > 0) first_key = query_position - window + 1;
+  const int first_key = first_visible_key(query_position, window);
   if (((run + 1) * PA_RUN <= first_key && run * PA_RUN >= kept) || run * PA_RUN > query_position) return;   // no key of this run is visible
   const int kvh = head / (Hq / Hkv);
   const int tid = threadIdx.x;
@@ -513,8 +517,7 @@ paged_attention_tile_kernel(const T* __restrict__ q, long q_ld, int Hq, int Hkv,
   if (count <= 0) return;
   const int last_position = positions[first_row + count - 1];      // positions ascend within a lane
   const int first_position = positions[first_row];
-  int tile_first_key = 0;                                           // the oldest key any query of the tile sees
-  if (window > 0 && first_position - window + 1 > 0) tile_first_key = first_position - window + 1;
+  const int tile_first_key = first_visible_key(first_position, window);     // the oldest key any query of the tile sees
   if (run * PA_RUN > last_position || ((run + 1) * PA_RUN <= tile_first_key && run * PA_RUN >= kept)) return;
   const int kvh = head / (Hq / Hkv);
   const int tid = threadIdx.x;
@@ -536,11 +539,12 @@ paged_attention_tile_kernel(const T* __restrict__ q, long q_ld, int Hq, int Hkv,
 #pragma unroll
       for (int d = 0; d < DIMS; ++d) group_o[i][g][d] = 0.f;
     }
-  int query_position[PT_PER_WAVE];
+  int query_position[PT_PER_WAVE], query_first[PT_PER_WAVE];
 #pragma unroll
   for (int i = 0; i < PT_PER_WAVE; ++i) {
     const int query = wave + i * PA_WAVES;
     query_position[i] = query < count ? positions[first_row + query] : -1;
+    query_first[i] = first_visible_key(max(query_position[i], 0), window);
   }
 
   // one group of 64 keys; called with a constant group so that what a wave keeps of it stays in registers
@@ -610,8 +614,7 @@ paged_attention_tile_kernel(const T* __restrict__ q, long q_ld, int Hq, int Hkv,
 #pragma unroll
     for (int i = 0; i < PT_PER_WAVE; ++i) {
       const int position = query_position[i];
-      int first_key = 0;
-      if (window > 0 && position - window + 1 > 0) first_key = position - window + 1;
+      const int first_key = query_first[i];
       const int key = group_first + lane;
       const bool visible = (key >= first_key || key < kept) && key <= position;
       float score = -INFINITY;
@@ -689,8 +692,7 @@ paged_attention_tile_kernel(const T* __restrict__ q, long q_ld, int Hq, int Hkv,
 #pragma unroll
   for (int i = 0; i < PT_PER_WAVE; ++i) {
     const int position = query_position[i];
-    int first_key = 0;
-    if (window > 0 && position - window + 1 > 0) first_key = position - window + 1;
+    const int first_key = query_first[i];
     if (position < 0 || ((run + 1) * PA_RUN <= first_key && run * PA_RUN >= kept) || run * PA_RUN > position) continue;    // the per-token kernel writes nothing either
     float best = group_max[i][0];
 #pragma unroll
@@ -725,12 +727,12 @@ template <typename T, bool FAST_EXP>
 __global__ void paged_attention_merge_kernel(const float* __restrict__ partial, int Hq, int dh, int runs,
                                              const int* __restrict__ positions, int window, int kept,
                                              const float* __restrict__ sinks, float fixed_sink, int has_fixed_sink,
-                                             T* __restrict__ out, long out_ld, int sigmoid) {
+                                             T* __restrict__ out, long out_ld, int sigmoid, const T* __restrict__ gate,
+                                             long gate_ld) {
   const long token = blockIdx.x;
   const int head = blockIdx.y;
   const int query_position = positions[token];
-  int first_key = 0;
-  if (window > 0 && query_position - window + 1 > 0) first_key = query_position - window + 1;
+  const int first_key = first_visible_key(query_position, window);
   const int first_run = first_key / PA_RUN;
   // a caller's bound on the contexts sizes the work area: a token beyond that bound merges the runs that
   // were launched for it and never reads outside the area
@@ -756,7 +758,8 @@ __global__ void paged_attention_merge_kernel(const float* __restrict__ partial, 
       denominator = denominator * keep + (FAST_EXP ? __expf(sink - larger) : expf(sink - larger));
       sum *= keep;
     }
-    out[token * out_ld + (long)head * dh + dim] = from_float<T>(sigmoid ? sum : sum / denominator);
+    const float gated = (sigmoid ? sum : sum / denominator) * output_gate(gate, gate_ld, token, (long)head * dh + dim);
+    out[token * out_ld + (long)head * dh + dim] = from_float<T>(gated);
   }
 }
 
@@ -801,8 +804,9 @@ extern "C" int mi_paged_attention(const void* q, int dtype, long q_ld, int T, in
                                   const float* log_bias, const float* sinks, float fixed_sink, int has_fixed_sink,
                                   int max_seq_len, float* partial, long partial_floats, void* out, long out_ld,
                                   const int* query_tiles, int num_tiles, int tile_tokens, const int* cu_seqlens,
-                                  const float* head_scales, const float* score_bias, int sigmoid,
-                                  hipStream_t stream) {
+                                  const float* head_scales, const float* score_bias, int sigmoid, const void* gate,
+                                  long gate_ld, hipStream_t stream) {
+  if (gate && gate_ld < (long)Hq * dv) return ERR_BAD_ARGUMENT;
   if ((score_bias && !sigmoid) || (sigmoid && (sinks || has_fixed_sink)) || (sinks && has_fixed_sink)) return ERR_BAD_ARGUMENT;
   if (kept < 0 || (kept > 0 && window <= 0)) return ERR_BAD_ARGUMENT;
   if (T <= 0 || Hq <= 0 || Hkv <= 0 || Hq % Hkv != 0 || dh <= 0 || dv <= 0 || page_size <= 0 || max_pages <= 0 ||
@@ -858,7 +862,8 @@ extern "C" int mi_paged_attention(const void* q, int dtype, long q_ld, int T, in
     }
     RETURN_IF_LAUNCH_FAILED();
     paged_attention_merge_kernel<float, false><<<merge_grid, merge_threads, 0, stream>>>(
-        partial, Hq, dv, runs, positions, window, kept, sinks, fixed_sink, has_fixed_sink, (float*)out, out_ld, sigmoid);
+        partial, Hq, dv, runs, positions, window, kept, sinks, fixed_sink, has_fixed_sink, (float*)out, out_ld, sigmoid,
+        (const float*)gate, gate_ld);
   } else if (dtype == DT_BF16) {
     if (tiled && dims == 1) TILE_LAUNCH(bf16_t, true, 1);
     else if (tiled && dims == 2) TILE_LAUNCH(bf16_t, true, 2);
@@ -878,7 +883,8 @@ extern "C" int mi_paged_attention(const void* q, int dtype, long q_ld, int T, in
     }
     RETURN_IF_LAUNCH_FAILED();
     paged_attention_merge_kernel<bf16_t, true><<<merge_grid, merge_threads, 0, stream>>>(
-        partial, Hq, dv, runs, positions, window, kept, sinks, fixed_sink, has_fixed_sink, (bf16_t*)out, out_ld, sigmoid);
+        partial, Hq, dv, runs, positions, window, kept, sinks, fixed_sink, has_fixed_sink, (bf16_t*)out, out_ld, sigmoid,
+        (const bf16_t*)gate, gate_ld);
   } else {
     return ERR_BAD_ARGUMENT;
   }
@@ -907,7 +913,8 @@ struct alignas(16) bf16x8 {
 };
 
 // dv: the width of a value head and of a head's output (any width; the keys' when it is DH).  head_scales
-// (a multiplier on a head's scores, after `scale`) and score_bias may be null.  sigmoid: a visible key weighs
+// (a multiplier on a head's scores, after `scale`), score_bias and slopes (score -= slopes[head] * distance) may be null.
+// dh: the width of a key head, a multiple of 8 up to DH (the lanes of a key's row past it bring nothing).  sigmoid: a visible key weighs
 // sigmoid(score + score_bias[head]) on its own; the block then records (0, 1) as its (max, sum) and the merge adds
 // the partial outputs as they are.  Dynamic LDS: DEC_WAVES * G * dv floats.
 // kept > 0 (with a window): the keys at positions below kept stay visible; those that lie before the window's first
@@ -920,8 +927,8 @@ decode_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, const b
                         const int* __restrict__ block_tables, int max_pages,
                         const int* __restrict__ lane_of_token, const int* __restrict__ positions, float scale,
                         int window, int split_keys, int splits, float* __restrict__ partial_o,
-                        float* __restrict__ partial_ml, int dv, const float* __restrict__ head_scales,
-                        const float* __restrict__ score_bias, int sigmoid, int kept) {
+                        float* __restrict__ partial_ml, int dh, int dv, const float* __restrict__ head_scales,
+                        const float* __restrict__ score_bias, const float* __restrict__ slopes, int sigmoid, int kept) {
   constexpr int LPR = DH / 8;
   constexpr int KPW = WAVE / LPR;
   constexpr int KPB = KPW * DEC_WAVES;
@@ -933,8 +940,7 @@ decode_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, const b
   const int kvh = blockIdx.y;
   const long token = blockIdx.z;
   const int pos = positions[token];
-  int first_key = 0;
-  if (window > 0 && pos - window + 1 > 0) first_key = pos - window + 1;
+  const int first_key = first_visible_key(pos, window);
   const int first_page_key = (first_key / page_size) * page_size;
   const bool kept_block = split == splits;                   // only launched with kept > 0
   const int stride = kept > 0 ? splits + 1 : splits;         // partial results of a head
@@ -960,12 +966,20 @@ decode_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, const b
   const int c = lane % LPR;
 
   float qf[G][8];
-  float offset_of[G];
+  float offset_of[G], slope_of[G];
+  const bool brings = c * 8 < dh;                // whether this lane's piece of a key's row exists
 #pragma unroll
   for (int g = 0; g < G; ++g) {
-    const bf16x8 packed = *reinterpret_cast<const bf16x8*>(q + token * q_ld + (long)(kvh * G + g) * DH + c * 8);
     const float factor = head_scales ? scale * head_scales[kvh * G + g] : scale;
     offset_of[g] = score_bias ? score_bias[kvh * G + g] : 0.f;
+    slope_of[g] = slopes ? slopes[kvh * G + g] : 0.f;
+    bf16x8 packed;
+    if (brings) {
+      packed = *reinterpret_cast<const bf16x8*>(q + token * q_ld + (long)(kvh * G + g) * dh + c * 8);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) packed.v[j] = (bf16_t)0.f;
+    }
 #pragma unroll
     for (int j = 0; j < 8; ++j) qf[g][j] = (float)packed.v[j] * factor;
   }
@@ -978,11 +992,11 @@ decode_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, const b
     float s[G];
 #pragma unroll
     for (int g = 0; g < G; ++g) s[g] = 0.f;
-    if (valid) {
+    if (valid && brings) {
       const int page = table[key / page_size];
       const int offset = key % page_size;
       const bf16x8 packed = *reinterpret_cast<const bf16x8*>(
-          k_base + (long)page * page_stride + ((long)kvh * page_size + offset) * DH + c * 8);
+          k_base + (long)page * page_stride + ((long)kvh * page_size + offset) * dh + c * 8);
       float kf[8];
 #pragma unroll
       for (int j = 0; j < 8; ++j) kf[j] = (float)packed.v[j];
@@ -997,7 +1011,10 @@ decode_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, const b
       for (int g = 0; g < G; ++g) s[g] += __shfl_xor(s[g], offset, WAVE);
     if (valid && c == 0) {
 #pragma unroll
-      for (int g = 0; g < G; ++g) s_lds[g][local] = (key >= first_key || key < kept) ? s[g] + offset_of[g] : -INFINITY;
+      for (int g = 0; g < G; ++g) {
+        const float score = fmaf(-slope_of[g], (float)(pos - key), s[g] + offset_of[g]);
+        s_lds[g][local] = (key >= first_key || key < kept) ? score : -INFINITY;
+      }
     }
   }
   __syncthreads();
@@ -1104,12 +1121,12 @@ decode_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, const b
 __global__ void decode_merge_kernel(const float* __restrict__ partial_o, const float* __restrict__ partial_ml,
                                     const int* __restrict__ positions, int window, int page_size,
                                     int split_keys, int splits, int Hq, int dh, bf16_t* __restrict__ out,
-                                    long out_ld, int sigmoid, int kept, const float* __restrict__ sinks) {
+                                    long out_ld, int sigmoid, int kept, const float* __restrict__ sinks,
+                                    const bf16_t* __restrict__ gate, long gate_ld) {
   const long token = blockIdx.x;
   const int head = blockIdx.y;
   const int pos = positions[token];
-  int first_key = 0;
-  if (window > 0 && pos - window + 1 > 0) first_key = pos - window + 1;
+  const int first_key = first_visible_key(pos, window);
   const int first_page_key = (first_key / page_size) * page_size;
   const int used = min(splits, (pos - first_page_key) / split_keys + 1);
   const int stride = kept > 0 ? splits + 1 : splits;
@@ -1120,7 +1137,7 @@ __global__ void decode_merge_kernel(const float* __restrict__ partial_o, const f
       float sum = 0.f;
       for (int s = 0; s < used; ++s) sum += o[(long)s * dh + dim];
       if (kept > 0) sum += o[(long)splits * dh + dim];
-      out[token * out_ld + (long)head * dh + dim] = (bf16_t)sum;
+      out[token * out_ld + (long)head * dh + dim] = (bf16_t)(sum * output_gate(gate, gate_ld, token, (long)head * dh + dim));
     }
     return;
   }
@@ -1138,7 +1155,7 @@ __global__ void decode_merge_kernel(const float* __restrict__ partial_o, const f
       float sum = 0.f;
       for (int s = 0; s < used; ++s) sum += __expf(ml[2 * s] - maximum) * o[(long)s * dh + dim];
       if (kept > 0) sum += kept_factor * o[(long)splits * dh + dim];
-      out[token * out_ld + (long)head * dh + dim] = (bf16_t)(sum / denominator);
+      out[token * out_ld + (long)head * dh + dim] = (bf16_t)(sum / denominator * output_gate(gate, gate_ld, token, (long)head * dh + dim));
     }
     return;
   }
@@ -1165,7 +1182,7 @@ __global__ void decode_merge_kernel(const float* __restrict__ partial_o, const f
     for (int dim = threadIdx.x; dim < dh; dim += blockDim.x) {
       float sum = 0.f;
       for (int s = 0; s < used; ++s) sum = fmaf(factor_lds[s], o[(long)s * dh + dim], sum);
-      out[token * out_ld + (long)head * dh + dim] = (bf16_t)(sum / denominator);
+      out[token * out_ld + (long)head * dh + dim] = (bf16_t)(sum / denominator * output_gate(gate, gate_ld, token, (long)head * dh + dim));
     }
     return;
   }
@@ -1176,7 +1193,7 @@ __global__ void decode_merge_kernel(const float* __restrict__ partial_o, const f
   for (int dim = threadIdx.x; dim < dh; dim += blockDim.x) {
     float sum = 0.f;
     for (int s = 0; s < used; ++s) sum += __expf(ml[2 * s] - maximum) * o[(long)s * dh + dim];
-    out[token * out_ld + (long)head * dh + dim] = (bf16_t)(sum / denominator);
+    out[token * out_ld + (long)head * dh + dim] = (bf16_t)(sum / denominator * output_gate(gate, gate_ld, token, (long)head * dh + dim));
   }
 }
 
@@ -1184,18 +1201,19 @@ template <int DH, int G>
 static int launch_decode(const bf16_t* q, long q_ld, int T, int Hq, int Hkv, const bf16_t* k_base,
                          const bf16_t* v_base, long page_stride, int page_size, const int* block_tables,
                          int max_pages, const int* lane_of_token, const int* positions, float scale, int window,
-                         int split_keys, int splits, float* partial_o, float* partial_ml, int dv,
-                         const float* head_scales, const float* score_bias, int sigmoid, int kept, hipStream_t stream) {
+                         int split_keys, int splits, float* partial_o, float* partial_ml, int dh, int dv,
+                         const float* head_scales, const float* score_bias, const float* slopes, int sigmoid, int kept,
+                         hipStream_t stream) {
   const dim3 grid(kept > 0 ? splits + 1 : splits, Hkv, T);
   const size_t dynamic = sizeof(float) * DEC_WAVES * G * (size_t)dv;
   decode_attention_kernel<DH, G><<<grid, DEC_THREADS, dynamic, stream>>>(
       q, q_ld, Hq, k_base, v_base, page_stride, page_size, block_tables, max_pages, lane_of_token, positions,
-      scale, window, split_keys, splits, partial_o, partial_ml, dv, head_scales, score_bias, sigmoid, kept);
+      scale, window, split_keys, splits, partial_o, partial_ml, dh, dv, head_scales, score_bias, slopes, sigmoid, kept);
   return 0;
 }
 
 // Returns ERR_UNSUPPORTED_SIZE for shapes this kernel does not cover (the caller then uses
-// mi_paged_attention): head_dim 64 or 128, 1..8 query heads per kv head, page_size a multiple of 8,
+// mi_paged_attention): head_dim a multiple of 8 up to 128, 1..8 query heads per kv head, page_size a multiple of 8,
 // split_keys a multiple of page_size and at most DEC_MAX_SPLIT, values of up to 256 dims a head.
 // partial_o holds T * Hq * splits * dv floats (with kept > 0: splits + 1 a head, and partial_ml likewise).
 // kept (with a window): the first keys that stay visible, at most DEC_MAX_SPLIT; sinks (float32 per query head, or
@@ -1205,23 +1223,26 @@ extern "C" int mi_decode_attention_forms(const void* q, long q_ld, int T, int Hq
                                          const int* block_tables, int max_pages, const int* lane_of_token,
                                          const int* positions, float scale, int window, int split_keys, int splits,
                                          float* partial_o, float* partial_ml, void* out, long out_ld,
-                                         const float* head_scales, const float* score_bias, int sigmoid,
-                                         int kept, const float* sinks, hipStream_t stream) {
+                                         const float* head_scales, const float* score_bias, const float* slopes,
+                                         int sigmoid, int kept, const float* sinks, const void* gate, long gate_ld,
+                                         hipStream_t stream) {
   if (T <= 0 || Hq <= 0 || Hkv <= 0 || Hq % Hkv != 0 || page_size <= 0 || splits <= 0 || max_pages <= 0 || dv <= 0)
     return ERR_BAD_ARGUMENT;
   if (kept < 0 || (kept > 0 && window <= 0) || (sinks && sigmoid)) return ERR_BAD_ARGUMENT;
+  if (gate && gate_ld < (long)Hq * dv) return ERR_BAD_ARGUMENT;
   if (kept > DEC_MAX_SPLIT) return ERR_UNSUPPORTED_SIZE;
   const int G = Hq / Hkv;
-  if ((dh != 64 && dh != 128) || G > 8 || page_size % 8 != 0 || split_keys % page_size != 0 ||
+  if (dh <= 0 || dh % 8 != 0 || dh > 128 || G > 8 || page_size % 8 != 0 || split_keys % page_size != 0 ||
       split_keys <= 0 || split_keys > DEC_MAX_SPLIT || T > 65535 || Hkv > 65535 || dv > 256)
     return ERR_UNSUPPORTED_SIZE;
   if (score_bias != nullptr && !sigmoid) return ERR_BAD_ARGUMENT;
+  const int lanes_width = dh <= 64 ? 64 : 128;
 #define DECODE_CASE(DH_, G_)                                                                                     \
-  if (dh == DH_ && G == G_)                                                                                      \
+  if (lanes_width == DH_ && G == G_)                                                                                      \
     launch_decode<DH_, G_>((const bf16_t*)q, q_ld, T, Hq, Hkv, (const bf16_t*)k_base, (const bf16_t*)v_base,     \
                            page_stride, page_size, block_tables, max_pages, lane_of_token, positions, scale,     \
-                           window, split_keys, splits, partial_o, partial_ml, dv, head_scales, score_bias,       \
-                           sigmoid, kept, stream);
+                           window, split_keys, splits, partial_o, partial_ml, dh, dv, head_scales, score_bias,   \
+                           slopes, sigmoid, kept, stream);
   DECODE_CASE(64, 1) DECODE_CASE(64, 2) DECODE_CASE(64, 3) DECODE_CASE(64, 4) DECODE_CASE(64, 5)
   DECODE_CASE(64, 6) DECODE_CASE(64, 7) DECODE_CASE(64, 8)
   DECODE_CASE(128, 1) DECODE_CASE(128, 2) DECODE_CASE(128, 3) DECODE_CASE(128, 4) DECODE_CASE(128, 5)
@@ -1232,7 +1253,7 @@ extern "C" int mi_decode_attention_forms(const void* q, long q_ld, int T, int Hq
   const int merge_threads = dv <= 64 ? 64 : dv <= 128 ? 128 : 256;
   decode_merge_kernel<<<merge_grid, merge_threads, 0, stream>>>(partial_o, partial_ml, positions, window, page_size,
                                                                 split_keys, splits, Hq, dv, (bf16_t*)out, out_ld,
-                                                                sigmoid, kept, sinks);
+                                                                sigmoid, kept, sinks, (const bf16_t*)gate, gate_ld);
   RETURN_IF_LAUNCH_FAILED();
   return 0;
 }
@@ -1245,7 +1266,7 @@ extern "C" int mi_decode_attention(const void* q, long q_ld, int T, int Hq, int 
                                    void* out, long out_ld, hipStream_t stream) {
   return mi_decode_attention_forms(q, q_ld, T, Hq, Hkv, dh, dh, k_base, v_base, page_stride, page_size, block_tables,
                                    max_pages, lane_of_token, positions, scale, window, split_keys, splits, partial_o,
-                                   partial_ml, out, out_ld, nullptr, nullptr, 0, 0, nullptr, stream);
+                                   partial_ml, out, out_ld, nullptr, nullptr, nullptr, 0, 0, nullptr, nullptr, 0, stream);
 }
 
 // ---------------------------------------------------------------- decode attention without a workspace argument
@@ -1301,200 +1322,7 @@ extern "C" int mi_decode_attention_static(const void* q, long q_ld, int T, int H
                              base + o_floats, out, out_ld, stream);
 }
 
-// ---------------------------------------------------------------- prefill attention on the matrix cores
-// bfloat16, head_dim 64 or 128.  grid = (4 x query tiles, kv heads, head passes): a tile is up to 64
-// consecutive tokens of one lane and a workgroup takes 16 of them with the query heads of one kv
-// head (NSET column sets that share every K and V fragment).  The keys, from the first visible
-// one to the workgroup's last position, are split in eight runs of whole 32-key steps, one per
-// wave, read straight from the cache pages (the portion's own keys were written by rope_kv_store
-// before), four steps in flight at a time; the eight partial results are merged through LDS,
-// set by set.  Workgroups with the longest contexts (the last tiles) are launched first, in every
-// other head pass last.
-#include "attn_mfma.h"
-
-#define PREFILL_STEPS 4
-#define PREFILL_WAVES 8
-#define PREFILL_FILL_BLOCKS 512   // two workgroups for each of the 256 compute units
-
-// EXTRAS: the scores lose log_bias[head] = (r1, r2) -> r1 * ln(1 + r2 * distance), and the softmax's denominator
-// holds one more term exp(sinks[head]) (either pointer may be null).
-// DV: the width the values are computed with, the keys' or, PADDED, the next width of the launch's table above
-// value_dim, the width of the cached values and of a head's output (a multiple of 4).
-// SIGMOID: a visible key weighs sigmoid(score * scale * head_scales[head] + score_bias[head]) on its own (either
-// pointer may be null: 1 and 0); no maximum, no normalizer, the waves' partial sums are added as they are.
-template <int DH, int NSET, bool EXTRAS = false, int DV = DH, bool SIGMOID = false, bool PADDED = false>
-__global__ void __launch_bounds__(PREFILL_WAVES * WAVE)
-prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hkv, const bf16_t* __restrict__ k_base,
-                         const bf16_t* __restrict__ v_base, long page_stride, int page_size,
-                         const int* __restrict__ block_tables, int max_pages, const int* __restrict__ tiles,
-                         const int* __restrict__ cu_seqlens, const int* __restrict__ start_pos, float scale,
-                         int window, bf16_t* __restrict__ out, long out_ld,
-                         const float* __restrict__ log_bias = nullptr, const float* __restrict__ sinks = nullptr,
-                         int value_dim = DV, const float* __restrict__ head_scales = nullptr,
-                         const float* __restrict__ score_bias = nullptr, int kept = 0) {
-  constexpr int ITEMS = 2 + 4 * (DV / 16);                    // m, l and the accumulator of one set
-  __shared__ float part[PREFILL_WAVES][ITEMS][WAVE];
-  __shared__ int wave_pages[PREFILL_WAVES][WAVE];
-  // heavy ones first; every other head pass the other way round, so that workgroups of two passes that
-  // run side by side bring about the same work together
-  const int block = (blockIdx.z & 1) ? blockIdx.x : gridDim.x - 1 - blockIdx.x;
-  const int tile = block / 4;
-  const int kvh = blockIdx.y;
-  const int G = Hq / Hkv;
-  const int head0 = kvh * G + blockIdx.z * NSET;             // first head of this pass
-  const int request = tiles[2 * tile];
-  if (request < 0) return;                                    // a row of the table past the step's own runs
-  const int lane = threadIdx.x & (WAVE - 1);
-  const int wave = threadIdx.x / WAVE;
-  const int qd = lane / 16;
-  const int n = lane % 16;
-  const int lane_end = cu_seqlens[request + 1];
-  const int first_token = tiles[2 * tile + 1] + 16 * (block % 4);
-  if (first_token >= lane_end) return;                        // the whole workgroup
-  const int token = first_token + n;
-  const bool has_query = token < lane_end;
-  const int base_position = start_pos[request] - cu_seqlens[request];
-  const int position = base_position + token;
-  const int last_position = base_position + min(first_token + 15, lane_end - 1);
-  const int first_position = base_position + first_token;
-  // every column of the wave holds a query (16 tokens, and the head sets divide the heads): the wave's bounds are known
-  const bool full_tile = first_token + 16 <= lane_end && (blockIdx.z + 1) * NSET <= G;
-
-  mfma_bf16x8 q_frag[NSET][DH / 32];
-  int col_pos[NSET];
-#pragma unroll
-  for (int s = 0; s < NSET; ++s) {
-    const bool valid = has_query && blockIdx.z * NSET + s < G;
-    col_pos[s] = valid ? position : -1;
-#pragma unroll
-    for (int kk = 0; kk < DH / 32; ++kk) {
-      if (valid) {
-        q_frag[s][kk] = *reinterpret_cast<const mfma_bf16x8*>(q + (long)token * q_ld + (long)(head0 + s) * DH +
-                                                               32 * kk + 8 * qd);
-      } else {
-#pragma unroll
-        for (int j = 0; j < 8; ++j) q_frag[s][kk][j] = (bf16_t)0.f;
-      }
-    }
-  }
-  AttnAccumulator<DH, NSET, DV> acc;
-  acc.clear();
-  AttnGate<NSET> gate;
-  if (SIGMOID) {
-#pragma unroll
-    for (int s = 0; s < NSET; ++s) {
-      const int head = min(head0 + s, Hq - 1);
-      gate.scale[s] = scale * (head_scales ? head_scales[head] : 1.f);
-      gate.bias[s] = score_bias ? score_bias[head] : 0.f;
-    }
-  }
-  AttnLogBias<NSET> bias;
-  if (EXTRAS) {
-    bias.on = log_bias != nullptr;
-#pragma unroll
-    for (int s = 0; s < NSET; ++s) {
-      const int head = min(head0 + s, Hq - 1);
-      bias.r1[s] = log_bias ? log_bias[2 * head] : 0.f;
-      bias.r2[s] = log_bias ? log_bias[2 * head + 1] : 0.f;
-    }
-  }
-  AttnCache cache;
-  cache.k_base = k_base;
-  cache.v_base = v_base;
-  cache.page_stride = page_stride;
-  cache.page_size = page_size;
-  cache.kvh = kvh;
-  cache.value_dim = value_dim;
-  const int* cache_pages = block_tables + (long)request * max_pages;
-  int key_lo = 0;
-  if (window > 0 && first_position - window + 1 > 0) key_lo = ((first_position - window + 1) / 32) * 32;
-  const int key_hi = last_position + 1;
-  const int steps = (key_hi - key_lo + 31) / 32;
-  const int steps_per_wave = (steps + PREFILL_WAVES - 1) / PREFILL_WAVES;
-  const int my_lo = key_lo + 32 * steps_per_wave * wave;
-  const int my_hi = min(key_hi, my_lo + 32 * steps_per_wave);
-  // the page ids of the run go through LDS, 64 pages at a time (a wave's own corner of it: no
-  // barrier), so that a K or V load does not wait for a load of its page id
-  auto walk = [&](int from, int to) {
-    for (int part_lo = from; part_lo < to;) {
-      const int first_page = part_lo / page_size;
-      const int part_hi = min(to, (first_page + WAVE) * page_size);
-      wave_pages[wave][lane] = cache_pages[min(first_page + lane, max_pages - 1)];
-      cache.pages = wave_pages[wave];
-      cache.base_page = first_page;
-      attend_keys<DH, NSET, PREFILL_STEPS, false, EXTRAS, DV, SIGMOID, PADDED>(
-          acc, q_frag, col_pos, window, scale, part_lo, part_hi, cache, full_tile ? first_position : -1, last_position,
-          bias, &gate, kept);
-      part_lo = part_hi;
-    }
-  };
-  walk(my_lo, my_hi);
-  // the kept first keys that lie before the window's first step: the last wave, whose own run is the shortest
-  if (kept > 0 && key_lo > 0 && wave == PREFILL_WAVES - 1) walk(0, min(kept, key_lo));
-
-  // merge: set s is finished by wave s
-#pragma unroll
-  for (int s = 0; s < NSET; ++s) {
-    __syncthreads();
-    part[wave][0][lane] = acc.m[s];
-    part[wave][1][lane] = acc.l[s];
-#pragma unroll
-    for (int dt = 0; dt < DV / 16; ++dt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) part[wave][2 + 4 * dt + i][lane] = acc.o[s][dt][i];
-    __syncthreads();
-    if (wave != s % PREFILL_WAVES) continue;
-    if (SIGMOID) {
-      if (col_pos[s] < 0) continue;
-      bf16_t* o = out + (long)token * out_ld + (long)(head0 + s) * value_dim;
-#pragma unroll
-      for (int dt = 0; dt < DV / 16; ++dt) {
-        mfma_bf16x4 packed;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          float value = 0.f;
-#pragma unroll
-          for (int w = 0; w < PREFILL_WAVES; ++w) value += part[w][2 + 4 * dt + i][lane];
-          packed[i] = (bf16_t)value;
-        }
-        if (!PADDED || 16 * dt + 4 * qd < value_dim) *reinterpret_cast<mfma_bf16x4*>(o + 16 * dt + 4 * qd) = packed;
-      }
-      continue;
-    }
-    float m = -INFINITY;
-#pragma unroll
-    for (int w = 0; w < PREFILL_WAVES; ++w) m = fmaxf(m, part[w][0][lane]);
-    // the sink, in the scores' units of log2: it may be the largest term
-    const float sink = (EXTRAS && sinks) ? sinks[min(head0 + s, Hq - 1)] * 1.4426950408889634f : -INFINITY;
-    m = fmaxf(m, sink);
-    float factor[PREFILL_WAVES];
-    float l = 0.f;
-#pragma unroll
-    for (int w = 0; w < PREFILL_WAVES; ++w) {
-      const float m_w = part[w][0][lane];
-      factor[w] = m_w == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_w - m);
-      l += part[w][1][lane] * factor[w];
-    }
-    l += __shfl_xor(l, 16, WAVE);
-    l += __shfl_xor(l, 32, WAVE);
-    if (EXTRAS && sinks) l += __builtin_amdgcn_exp2f(sink - m);       // once for the column: no key, no value
-    if (col_pos[s] < 0) continue;
-    const float inverse = 1.f / l;
-    bf16_t* o = out + (long)token * out_ld + (long)(head0 + s) * value_dim;
-#pragma unroll
-    for (int dt = 0; dt < DV / 16; ++dt) {
-      mfma_bf16x4 packed;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        float value = 0.f;
-#pragma unroll
-        for (int w = 0; w < PREFILL_WAVES; ++w) value += part[w][2 + 4 * dt + i][lane] * factor[w];
-        packed[i] = (bf16_t)(value * inverse);
-      }
-      if (!PADDED || 16 * dt + 4 * qd < value_dim) *reinterpret_cast<mfma_bf16x4*>(o + 16 * dt + 4 * qd) = packed;
-    }
-  }
-}
+#include "attn_prefill.h"
 
 // The widths the values are computed with when they are not the keys' (the cached width rounded up to one of them),
 // and the query heads that share a key fragment at that width: the accumulators of a set grow with it.
@@ -1563,7 +1391,9 @@ extern "C" int mi_prefill_attention(const void* q, long q_ld, int Hq, int Hkv, i
                                     int max_pages, const int* tiles, int n_tiles, const int* cu_seqlens,
                                     const int* start_pos, float scale, int window, int max_seq_len, void* out,
                                     long out_ld, const float* log_bias, const float* sinks, int kept,
-                                    hipStream_t stream) {
+                                    const float* slopes, const void* gate, long gate_ld, hipStream_t stream) {
+  if ((log_bias && slopes) || (gate && (gate_ld < (long)Hq * dh || gate_ld % 4 != 0 || (uintptr_t)gate % 8 != 0)))
+    return ERR_BAD_ARGUMENT;
   if (n_tiles <= 0 || Hq <= 0 || Hkv <= 0 || Hq % Hkv != 0 || page_size <= 0 || max_pages <= 0)
     return ERR_BAD_ARGUMENT;
   if (kept < 0 || (kept > 0 && window <= 0)) return ERR_BAD_ARGUMENT;      // first keys are kept behind a window
@@ -1583,19 +1413,19 @@ extern "C" int mi_prefill_attention(const void* q, long q_ld, int Hq, int Hkv, i
   const int nset = (G + passes - 1) / passes;
   if (n_tiles > (1 << 28)) return ERR_UNSUPPORTED_SIZE;
   const dim3 grid(4 * n_tiles, Hkv, passes);
-  const bool extras = log_bias != nullptr || sinks != nullptr;
+  const bool extras = log_bias != nullptr || sinks != nullptr || slopes != nullptr;
 #define PREFILL_CASE(DH_, NSET_)                                                                              \
   if (dh == DH_ && nset == NSET_) {                                                                           \
     if (extras)                                                                                               \
       prefill_attention_kernel<DH_, NSET_, true><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(                  \
           (const bf16_t*)q, q_ld, Hq, Hkv, (const bf16_t*)k_base, (const bf16_t*)v_base, page_stride, page_size, \
           block_tables, max_pages, tiles, cu_seqlens, start_pos, scale, window, (bf16_t*)out, out_ld, log_bias, sinks, \
-          DH_, nullptr, nullptr, kept);                                                                       \
+          DH_, nullptr, nullptr, kept, slopes, (const bf16_t*)gate, gate_ld);                                 \
     else                                                                                                      \
       prefill_attention_kernel<DH_, NSET_><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(                        \
           (const bf16_t*)q, q_ld, Hq, Hkv, (const bf16_t*)k_base, (const bf16_t*)v_base, page_stride, page_size, \
           block_tables, max_pages, tiles, cu_seqlens, start_pos, scale, window, (bf16_t*)out, out_ld, nullptr, \
-          nullptr, DH_, nullptr, nullptr, kept);                                                              \
+          nullptr, DH_, nullptr, nullptr, kept, nullptr, (const bf16_t*)gate, gate_ld);                       \
   }
   PREFILL_CASE(64, 1) PREFILL_CASE(64, 2) PREFILL_CASE(64, 3) PREFILL_CASE(64, 4)
   PREFILL_CASE(128, 1) PREFILL_CASE(128, 2) PREFILL_CASE(128, 3) PREFILL_CASE(128, 4)

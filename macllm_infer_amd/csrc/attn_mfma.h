@@ -15,7 +15,8 @@
 //            softmax (4 keys of tile 0, 4 keys of tile 1) are exactly its B fragment once the
 //            32 keys of the step are numbered (q, j) -> j < 4 ? 4q + j : 16 + 4q + (j - 4).
 // Formulas: s = q.k * scale, key visible when key <= column position and, with a window w,
-// position - key < w (reference: src/decoder.rs:4515-4532, 4641-4670) or, with kept > 0, key < kept (the first
+// position - key < w (reference: src/decoder.rs:4515-4532, 4641-4670; a negative w: keys of the column's own chunk of
+// -w positions, see first_visible_key) or, with kept > 0, key < kept (the first
 // keys of a sequence stay visible behind the window); softmax in float32.
 #pragma once
 #include "common.h"
@@ -117,12 +118,15 @@ __device__ __forceinline__ void attn_load(AttnFragments<DH, STEPS, DV>& f, int k
 
 // A bias on the scores that grows with the logarithm of the distance: score -= r1 * ln(1 + r2 * (position - key)),
 // one (r1, r2) for each set of columns (a query head).  In units of log2, where the scores live, that is
-// r1 * log2(1 + r2 * distance).  ``on`` false: no bias (the kernels that know none pass the default).
+// r1 * log2(1 + r2 * distance).  ``linear``: a bias that grows with the distance itself, score -= slope * distance
+// (``slope`` in units of log2).  Neither: no bias (the kernels that know none pass the default).
 template <int NSET>
 struct AttnLogBias {
   bool on = false;
+  bool linear = false;
   float r1[NSET];
   float r2[NSET];
+  float slope[NSET];
 };
 
 // Weights that are no softmax: a visible key weighs sigmoid(score * scale[set] + bias[set]) on its own, one pair
@@ -141,7 +145,7 @@ struct AttnGate {
 template <int DH, int NSET, int STEPS, bool MASKED = true, bool BIASED = false, int DV = DH, bool SIGMOID = false>
 __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc, AttnFragments<DH, STEPS, DV>& f,
                                              const mfma_bf16x8 (&q_frag)[NSET][DH / 32],
-                                             const int (&col_pos)[NSET], int window, float scale, int k00,
+                                             const int (&col_pos)[NSET], const int (&col_first)[NSET], float scale, int k00,
                                              int key_hi, const AttnLogBias<NSET>& bias = AttnLogBias<NSET>(),
                                              const AttnGate<NSET>* gate = nullptr, int kept = 0) {
   const int lane = threadIdx.x & (WAVE - 1);
@@ -191,6 +195,12 @@ __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc,
               const float distance = (float)(col_pos[s] - (k0 + 16 * t + 4 * q + i));
               score[t][i] = fmaf(score[t][i], scale_log2, -bias.r1[s] * __log2f(fmaf(bias.r2[s], fmaxf(distance, 0.f), 1.f)));
             }
+        } else if (bias.linear) {
+#pragma unroll
+          for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+              score[t][i] = fmaf(score[t][i], scale_log2, -bias.slope[s] * (float)(col_pos[s] - (k0 + 16 * t + 4 * q + i)));
         } else {                       // a caller of this form for its sink alone: the scale, no logarithms
 #pragma unroll
           for (int t = 0; t < 2; ++t)
@@ -203,7 +213,7 @@ __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc,
         // they are lo .. lo + span, so one unsigned compare per score decides (an empty range gets
         // a lo that no offset reaches)
         const int position = col_pos[s];
-        const int first_visible = window > 0 ? max(position - window + 1, 0) : 0;
+        const int first_visible = col_first[s];
         const int last_visible = min(position, last_key);
         const bool any = last_visible >= first_visible;
         const int lo = any ? first_visible - k0 : 0x40000000;
@@ -270,7 +280,7 @@ __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc,
 // Keys [key_lo, key_hi): key_lo a multiple of 4; every key < key_hi is in the cache.
 // q_frag[s][kk]: lane (q, n) holds Q[column n of set s][dims 32*kk + 8q .. +8].
 // col_pos[s]: the position of lane's column n in set s (its last visible key), or -1 for a
-// column that holds no query.  window: 0 = none.  STEPS: 32-key steps whose loads are all
+// column that holds no query.  window: 0 = none, negative = chunks (first_visible_key).  STEPS: 32-key steps whose loads are all
 // requested before the first is used.  PIPELINED: the loads of the next STEPS steps are
 // requested before the current ones are worked on (twice the fragment registers), for callers
 // with long runs; a caller whose run is one round of STEPS steps gains nothing from it.
@@ -288,6 +298,9 @@ __device__ __forceinline__ void attend_keys(AttnAccumulator<DH, NSET, DV>& acc,
                                             const AttnGate<NSET>* gate = nullptr, int kept = 0) {
   const int last_key = key_hi - 1;
   constexpr int ROUND = 32 * STEPS;
+  int col_first[NSET];                 // the first key each column sees
+#pragma unroll
+  for (int s = 0; s < NSET; ++s) col_first[s] = first_visible_key(max(col_pos[s], 0), window);
   if (PIPELINED) {
     // the next round is always asked for, also past the end of the run (its keys are clamped to
     // the last one and never used): a condition around the loads would cost a wait
@@ -295,27 +308,27 @@ __device__ __forceinline__ void attend_keys(AttnAccumulator<DH, NSET, DV>& acc,
     attn_load<DH, STEPS, DV>(even, key_lo, last_key, cache);
     for (int k00 = key_lo; k00 < key_hi; k00 += 2 * ROUND) {
       attn_load<DH, STEPS, DV>(odd, k00 + ROUND, last_key, cache);
-      attn_compute<DH, NSET, STEPS, true, false, DV>(acc, even, q_frag, col_pos, window, scale, k00, key_hi);
+      attn_compute<DH, NSET, STEPS, true, false, DV>(acc, even, q_frag, col_pos, col_first, scale, k00, key_hi);
       attn_load<DH, STEPS, DV>(even, k00 + 2 * ROUND, last_key, cache);
       if (k00 + ROUND < key_hi)
-        attn_compute<DH, NSET, STEPS, true, false, DV>(acc, odd, q_frag, col_pos, window, scale, k00 + ROUND, key_hi);
+        attn_compute<DH, NSET, STEPS, true, false, DV>(acc, odd, q_frag, col_pos, col_first, scale, k00 + ROUND, key_hi);
     }
   } else {
     // rounds all of whose keys every column of the wave sees run without masks, in a loop of
     // their own; the rest (the diagonal, a window's edge, the end of the run) with them
     int open_hi = key_lo;
-    if (min_pos >= 0 && (window <= 0 || key_lo >= max_pos - window + 1))
+    if (min_pos >= 0 && key_lo >= first_visible_key(max_pos, window))
       open_hi = key_lo + max(0, (min(min_pos + 1, key_hi) - key_lo) / ROUND) * ROUND;
     for (int k00 = key_lo; k00 < open_hi; k00 += ROUND) {
       AttnFragments<DH, STEPS, DV> f;
       attn_load<DH, STEPS, DV, PADDED, PADDED_KEYS>(f, k00, last_key, cache);
-      attn_compute<DH, NSET, STEPS, false, BIASED, DV, SIGMOID>(acc, f, q_frag, col_pos, window, scale, k00, key_hi, bias,
+      attn_compute<DH, NSET, STEPS, false, BIASED, DV, SIGMOID>(acc, f, q_frag, col_pos, col_first, scale, k00, key_hi, bias,
                                                                 gate);
     }
     for (int k00 = open_hi; k00 < key_hi; k00 += ROUND) {
       AttnFragments<DH, STEPS, DV> f;
       attn_load<DH, STEPS, DV, PADDED, PADDED_KEYS>(f, k00, last_key, cache);
-      attn_compute<DH, NSET, STEPS, true, BIASED, DV, SIGMOID>(acc, f, q_frag, col_pos, window, scale, k00, key_hi, bias,
+      attn_compute<DH, NSET, STEPS, true, BIASED, DV, SIGMOID>(acc, f, q_frag, col_pos, col_first, scale, k00, key_hi, bias,
                                                                gate, kept);
     }
   }

@@ -60,6 +60,21 @@ __device__ __forceinline__ float tanh_norm_f(float x, float alpha, float weight,
   return fmaf(tanhf(alpha * x), weight, bias);
 }
 
+// The first key that a query at `position` sees.  span > 0: a window, the span most recent keys; span < 0: chunks of
+// -span positions counted from the sequence's start, of which a query sees its own; 0: every key up to its own.
+__host__ __device__ __forceinline__ int first_visible_key(int position, int span) {
+  if (span > 0) return position - span + 1 > 0 ? position - span + 1 : 0;
+  if (span < 0) return position - position % -span;
+  return 0;
+}
+
+// A gate on the heads' outputs: every attention kernel's last stage multiplies what it writes by sigmoid(gate) where the step has one: a row of
+// `gate` (row stride gate_ld, the activation type) holds one number for every dim of every head's output.
+template <typename T>
+__device__ __forceinline__ float output_gate(const T* gate, long gate_ld, long token, long column) {
+  return gate ? 1.0f / (1.0f + expf(-to_float(gate[token * gate_ld + column]))) : 1.0f;
+}
+
 #define RETURN_IF_LAUNCH_FAILED()                 \
   do {                                            \
     hipError_t launch_error_ = hipGetLastError(); \

@@ -26,6 +26,38 @@ extern "C" int mi_embed(const int* ids, const void* table, int table_dtype, floa
   return 0;
 }
 
+// The same through an RMS norm on the way into the stream: e = table[ids[t], :] * multiplier,
+// h[t, :] = e / sqrt(mean(e^2) + eps) * weight.  One workgroup a token; the row is read twice, the second time from a cache.
+template <typename T>
+__global__ void __launch_bounds__(256)
+embed_rmsnorm_kernel(const int* __restrict__ ids, const T* __restrict__ table, float multiplier,
+                     const float* __restrict__ weight, float eps, float* __restrict__ h, int d) {
+  __shared__ float scratch[16];
+  const long token = blockIdx.x;
+  const T* row = table + (long)ids[token] * d;
+  float* out = h + token * d;
+  float squares = 0.f;
+  for (int i = threadIdx.x; i < d; i += blockDim.x) {
+    const float e = to_float(row[i]) * multiplier;
+    squares = fmaf(e, e, squares);
+  }
+  const float rms = sqrtf(block_sum(squares, scratch) / (float)d + eps);
+  for (int i = threadIdx.x; i < d; i += blockDim.x) out[i] = to_float(row[i]) * multiplier / rms * weight[i];
+}
+
+extern "C" int mi_embed_rmsnorm(const int* ids, const void* table, int table_dtype, float multiplier, const float* weight,
+                                float eps, float* h, int T, int d, hipStream_t stream) {
+  if (!ids || !table || !weight || !h || T <= 0 || d <= 0) return ERR_BAD_ARGUMENT;
+  if (table_dtype == DT_F32)
+    embed_rmsnorm_kernel<float><<<T, 256, 0, stream>>>(ids, (const float*)table, multiplier, weight, eps, h, d);
+  else if (table_dtype == DT_BF16)
+    embed_rmsnorm_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, (const bf16_t*)table, multiplier, weight, eps, h, d);
+  else
+    return ERR_BAD_ARGUMENT;
+  RETURN_IF_LAUNCH_FAILED();
+  return 0;
+}
+
 // ---------------------------------------------------------------- tokens fed from the device
 // token_ids[dst[i]] = source[src[i]]: the tokens that the sampler left on the device for the step before go
 // into this step's token ids without a round trip through the host (the host learns them one step late).
@@ -399,7 +431,8 @@ __device__ __forceinline__ long swiglu_gate_at(int i, int I, int tile) {
   return tile == 0 ? i : (long)(i / tile) * 2 * tile + i % tile;
 }
 
-// the gate's activation: 0 SiLU, 1 the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))
+// the gate's activation: 0 SiLU, 1 the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), 2 the clamped
+// gated activation g sigmoid(alpha g) (u + offset) with g = min(gate, limit), u = clamp(up, -limit, limit)
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
@@ -409,9 +442,25 @@ __device__ __forceinline__ float gelu_tanh_bf16_f(float z) {
   return z * (1.0f - __frcp_rn(1.0f + __expf(2.0f * y)));
 }
 
+struct GluNumbers {
+  float limit, alpha, offset;
+};
+
+__device__ __forceinline__ float clamped_glu_f(float gate, float up, float limit, float alpha, float offset) {
+  const float g = fminf(gate, limit);
+  const float u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.0f + expf(-alpha * g)) * (u + offset);
+}
+// the same with the hardware's exponential and reciprocal; for results rounded to bfloat16 at once
+__device__ __forceinline__ float clamped_glu_bf16_f(float gate, float up, float limit, float alpha, float offset) {
+  const float g = fminf(gate, limit);
+  const float u = fminf(fmaxf(up, -limit), limit);
+  return g * __frcp_rn(1.0f + __expf(-alpha * g)) * (u + offset);
+}
+
 template <typename T>
 __global__ void swiglu_kernel(const T* __restrict__ gu, long ld, T* __restrict__ out, int I, int tile, long total,
-                              int activation) {
+                              int activation, GluNumbers glu) {
   const long index = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (index >= total) return;
   const long t = index / I;
@@ -419,14 +468,15 @@ __global__ void swiglu_kernel(const T* __restrict__ gu, long ld, T* __restrict__
   const long at = swiglu_gate_at(i, I, tile);
   const float gate = to_float(gu[t * ld + at]);
   const float up = to_float(gu[t * ld + at + (tile == 0 ? I : tile)]);
-  out[index] = from_float<T>((activation == 1 ? gelu_tanh_f(gate) : silu_f(gate)) * up);
+  if (activation == 2) out[index] = from_float<T>(clamped_glu_f(gate, up, glu.limit, glu.alpha, glu.offset));
+  else out[index] = from_float<T>((activation == 1 ? gelu_tanh_f(gate) : silu_f(gate)) * up);
 }
 
 // bfloat16, eight elements a thread (I, ld and the addresses multiples of 8 elements; tile 0 or 8)
 typedef __bf16 common_bf16x8 __attribute__((ext_vector_type(8)));
 __global__ void __launch_bounds__(256)
 swiglu_vec_kernel(const bf16_t* __restrict__ gu, long ld, bf16_t* __restrict__ out, int I, int tile, long total,
-                  int activation) {
+                  int activation, GluNumbers glu) {
   const long index = ((long)blockIdx.x * blockDim.x + threadIdx.x) * 8;
   if (index >= total) return;
   const long t = index / I;
@@ -435,6 +485,13 @@ swiglu_vec_kernel(const bf16_t* __restrict__ gu, long ld, bf16_t* __restrict__ o
   const common_bf16x8 gate = *reinterpret_cast<const common_bf16x8*>(gu + t * ld + at);
   const common_bf16x8 up = *reinterpret_cast<const common_bf16x8*>(gu + t * ld + at + (tile == 0 ? I : 8));
   common_bf16x8 result;
+  if (activation == 2) {
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      result[j] = (bf16_t)clamped_glu_bf16_f((float)gate[j], (float)up[j], glu.limit, glu.alpha, glu.offset);
+    *reinterpret_cast<common_bf16x8*>(out + index) = result;
+    return;
+  }
 #pragma unroll
   for (int j = 0; j < 8; ++j)
     result[j] = (bf16_t)((activation == 1 ? gelu_tanh_bf16_f((float)gate[j]) : silu_bf16_f((float)gate[j])) * (float)up[j]);
@@ -442,19 +499,20 @@ swiglu_vec_kernel(const bf16_t* __restrict__ gu, long ld, bf16_t* __restrict__ o
 }
 
 extern "C" int mi_swiglu(const void* gu, int dtype, long ld, void* out, int T, int I, int tile, int activation,
-                         hipStream_t stream) {
-  if (T <= 0 || I <= 0 || ld < 2L * I || tile < 0 || (tile > 0 && I % tile != 0) || (activation != 0 && activation != 1))
+                         float limit, float alpha, float offset, hipStream_t stream) {
+  const GluNumbers glu = {limit, alpha, offset};
+  if (T <= 0 || I <= 0 || ld < 2L * I || tile < 0 || (tile > 0 && I % tile != 0) || activation < 0 || activation > 2)
     return ERR_BAD_ARGUMENT;
   const long total = (long)T * I;
   const int blocks = (int)((total + 255) / 256);
   if (dtype == DT_BF16 && I % 8 == 0 && ld % 8 == 0 && (tile == 0 || tile == 8) && ((uintptr_t)gu % 16) == 0 &&
       ((uintptr_t)out % 16) == 0) {
     const int vec_blocks = (int)((total / 8 + 255) / 256);
-    swiglu_vec_kernel<<<vec_blocks, 256, 0, stream>>>((const bf16_t*)gu, ld, (bf16_t*)out, I, tile, total, activation);
+    swiglu_vec_kernel<<<vec_blocks, 256, 0, stream>>>((const bf16_t*)gu, ld, (bf16_t*)out, I, tile, total, activation, glu);
   } else if (dtype == DT_F32)
-    swiglu_kernel<float><<<blocks, 256, 0, stream>>>((const float*)gu, ld, (float*)out, I, tile, total, activation);
+    swiglu_kernel<float><<<blocks, 256, 0, stream>>>((const float*)gu, ld, (float*)out, I, tile, total, activation, glu);
   else if (dtype == DT_BF16)
-    swiglu_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, ld, (bf16_t*)out, I, tile, total, activation);
+    swiglu_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, ld, (bf16_t*)out, I, tile, total, activation, glu);
   else
     return ERR_BAD_ARGUMENT;
   RETURN_IF_LAUNCH_FAILED();
@@ -961,15 +1019,150 @@ extern "C" int mi_add_layernorm(float* h, const void* rows0, int dtype0, float f
   return 0;
 }
 
+// ---------------------------------------------------------------- residual add + RMS norm behind the branches
+// s = f0 b0 + f1 b1 + f2 b2; v = h + s / sqrt(mean(s^2) + branch_eps) * branch_weight (float32; written back to h unless rows
+// are gathered); out (if wanted) = v / sqrt(mean(v^2) + eps) * weight.  One workgroup a row, which stays in registers: a
+// thread keeps CHUNKS pieces of VEC neighbouring elements (piece threadIdx.x + k * blockDim.x), and everything the later
+// stages read from memory is asked for at the start, beside the branches' rows.
+template <int VEC>
+__device__ __forceinline__ void floats_at(const float* from, float (&to)[VEC]) {
+  if constexpr (VEC == 4) {
+    const float4 piece = *reinterpret_cast<const float4*>(from);
+    to[0] = piece.x; to[1] = piece.y; to[2] = piece.z; to[3] = piece.w;
+  } else {
+    to[0] = from[0];
+  }
+}
+
+typedef __bf16 common_bf16x4 __attribute__((ext_vector_type(4)));
+
+template <int VEC>
+__device__ __forceinline__ void add_branch(const NormBranch& branch, long at, float (&to)[VEC]) {
+  if (!branch.rows) return;
+  if (branch.dtype == DT_BF16) {
+    if constexpr (VEC == 4) {
+      const common_bf16x4 piece = *reinterpret_cast<const common_bf16x4*>((const bf16_t*)branch.rows + at);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) to[j] += branch.factor * (float)piece[j];
+    } else {
+      to[0] += branch.factor * (float)((const bf16_t*)branch.rows)[at];
+    }
+    return;
+  }
+  float piece[VEC];
+  floats_at<VEC>((const float*)branch.rows + at, piece);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) to[j] += branch.factor * piece[j];
+}
+
+template <typename TO, int CHUNKS, int VEC>
+__global__ void __launch_bounds__(1024)
+add_normed_rmsnorm_kernel(float* __restrict__ h, NormBranch b0, NormBranch b1, NormBranch b2,
+                          const float* __restrict__ branch_weight, float branch_eps, const float* __restrict__ weight,
+                          float eps, TO* __restrict__ out, const int* __restrict__ rows, int d) {
+  __shared__ float scratch[16];
+  const long out_row = blockIdx.x;
+  const long row = rows ? (long)rows[out_row] : out_row;
+  float v[CHUNKS][VEC], branch[CHUNKS][VEC], bw[CHUNKS][VEC], w[CHUNKS][VEC];
+  float squares = 0.f;
+#pragma unroll
+  for (int k = 0; k < CHUNKS; ++k) {
+    const int i = (threadIdx.x + k * blockDim.x) * VEC;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[k][j] = branch[k][j] = bw[k][j] = w[k][j] = 0.f;
+    if (i < d) {
+      add_branch<VEC>(b0, row * d + i, branch[k]);
+      add_branch<VEC>(b1, row * d + i, branch[k]);
+      add_branch<VEC>(b2, row * d + i, branch[k]);
+      floats_at<VEC>(h + row * d + i, v[k]);
+      floats_at<VEC>(branch_weight + i, bw[k]);
+      if (out) floats_at<VEC>(weight + i, w[k]);
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) squares = fmaf(branch[k][j], branch[k][j], squares);
+  }
+  const float branch_rms = sqrtf(block_sum(squares, scratch) / (float)d + branch_eps);
+  squares = 0.f;
+#pragma unroll
+  for (int k = 0; k < CHUNKS; ++k) {
+    const int i = (threadIdx.x + k * blockDim.x) * VEC;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      v[k][j] = fmaf(branch[k][j] / branch_rms, bw[k][j], v[k][j]);
+      squares = fmaf(v[k][j], v[k][j], squares);
+    }
+    if (i < d && !rows) {
+      if constexpr (VEC == 4) *reinterpret_cast<float4*>(h + row * d + i) = make_float4(v[k][0], v[k][1], v[k][2], v[k][3]);
+      else h[row * d + i] = v[k][0];
+    }
+  }
+  if (!out) return;
+  const float rms = sqrtf(block_sum(squares, scratch) / (float)d + eps);
+  typedef TO four __attribute__((ext_vector_type(4)));
+#pragma unroll
+  for (int k = 0; k < CHUNKS; ++k) {
+    const int i = (threadIdx.x + k * blockDim.x) * VEC;
+    if (i >= d) continue;
+    if constexpr (VEC == 4) {
+      four piece;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) piece[j] = from_float<TO>(v[k][j] / rms * w[k][j]);
+      *reinterpret_cast<four*>(out + out_row * d + i) = piece;
+    } else {
+      out[out_row * d + i] = from_float<TO>(v[k][0] / rms * w[k][0]);
+    }
+  }
+}
+
+template <typename TO>
+static int launch_add_normed_rmsnorm(int n_rows, bool fours, hipStream_t stream, float* h, NormBranch b0, NormBranch b1,
+                                     NormBranch b2, const float* branch_weight, float branch_eps, const float* weight,
+                                     float eps, TO* out, const int* rows, int d) {
+  // few rows: as many threads as a row has pieces, for the shortest chain of waits; many rows: a few pieces a thread
+  const int pieces = fours ? d / 4 : d;
+  const int most = n_rows <= 512 ? 1024 : 256;
+  int chunks = 1;
+  while (chunks < 16 && (pieces + chunks - 1) / chunks > most) chunks *= 2;
+  const int threads = (((pieces + chunks - 1) / chunks + WAVE - 1) / WAVE) * WAVE;
+  if (threads > 1024) return ERR_UNSUPPORTED_SIZE;
+#define NORMED_CASE(CHUNKS_, VEC_)                                                                                     \
+  if (chunks == CHUNKS_ && fours == (VEC_ == 4))                                                                       \
+    add_normed_rmsnorm_kernel<TO, CHUNKS_, VEC_><<<n_rows, threads, 0, stream>>>(h, b0, b1, b2, branch_weight, branch_eps, \
+                                                                                 weight, eps, out, rows, d);
+  NORMED_CASE(1, 4) NORMED_CASE(2, 4) NORMED_CASE(4, 4) NORMED_CASE(8, 4) NORMED_CASE(16, 4)
+  NORMED_CASE(1, 1) NORMED_CASE(2, 1) NORMED_CASE(4, 1) NORMED_CASE(8, 1) NORMED_CASE(16, 1)
+#undef NORMED_CASE
+  return 0;
+}
+
+// d <= 16,384: sixteen elements for each of 1,024 threads (many rows: sixteen pieces of four for each of 256).
+extern "C" int mi_add_normed_rmsnorm(float* h, const void* rows0, int dtype0, float factor0, const void* rows1, int dtype1,
+                                     float factor1, const void* rows2, int dtype2, float factor2,
+                                     const float* branch_weight, float branch_eps, const float* weight, float eps,
+                                     void* out, int out_dtype, const int* rows, int n_rows, int d, hipStream_t stream) {
+  if (!h || !rows0 || !branch_weight || n_rows <= 0 || d <= 0 || (out && !weight) || (rows && !out)) return ERR_BAD_ARGUMENT;
+  if (d > 16384) return ERR_UNSUPPORTED_SIZE;
+  const NormBranch b0 = {rows0, dtype0, factor0}, b1 = {rows1, dtype1, factor1}, b2 = {rows2, dtype2, factor2};
+  const uintptr_t addresses = (uintptr_t)h | (uintptr_t)rows0 | (uintptr_t)rows1 | (uintptr_t)rows2 |
+                              (uintptr_t)branch_weight | (uintptr_t)weight | (uintptr_t)out;
+  const bool fours = d % 4 == 0 && addresses % 16 == 0;
+  int code;
+  if (out_dtype == DT_F32)
+    code = launch_add_normed_rmsnorm<float>(n_rows, fours, stream, h, b0, b1, b2, branch_weight, branch_eps, weight, eps,
+                                            (float*)out, rows, d);
+  else if (out_dtype == DT_BF16)
+    code = launch_add_normed_rmsnorm<bf16_t>(n_rows, fours, stream, h, b0, b1, b2, branch_weight, branch_eps, weight, eps,
+                                             (bf16_t*)out, rows, d);
+  else
+    return ERR_BAD_ARGUMENT;
+  if (code != 0) return code;
+  RETURN_IF_LAUNCH_FAILED();
+  return 0;
+}
+
 // ---------------------------------------------------------------- clamped gated activation
 // out[t, i] = g * sigmoid(alpha g) * (u + offset), g = min(gate, limit), u = clamp(up, -limit, limit); a row of
 // gate_up holds [gate | up].
-__device__ __forceinline__ float clamped_glu_f(float gate, float up, float limit, float alpha, float offset) {
-  const float g = fminf(gate, limit);
-  const float u = fminf(fmaxf(up, -limit), limit);
-  return g / (1.0f + expf(-alpha * g)) * (u + offset);
-}
-
 template <typename T>
 __global__ void clamped_glu_kernel(const T* __restrict__ gate_up, long ld, T* __restrict__ out, long out_ld, int I,
                                    long total, float limit, float alpha, float offset) {

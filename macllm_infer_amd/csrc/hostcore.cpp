@@ -76,7 +76,9 @@ struct Table {
 
 struct Group {
   int page_size;
-  int window;               // <= 0: every key is kept
+  // > 0: the window's most recent keys stay; < 0: the keys of the request's current chunk of -window positions stay;
+  // 0: every key is kept
+  int window;
   int kept_first = 0;       // with a window: keys at positions below this stay visible, their pages are never given back
   Pool pool;
   std::vector<Table> tables;   // by slot
@@ -213,8 +215,8 @@ int hc_reserve(void* handle, int n, const int* slots, const int* tokens, int* in
   return 0;
 }
 
-// The step ran: lengths advance, and a group with a window gives back every page all later
-// queries are past (the next query, at position `length`, sees keys >= length - window + 1).
+// The step ran: lengths advance, and a group with a window or chunks gives back every page all later queries are past
+// (the next query, at position `length`, sees keys >= length - window + 1, or those of its own chunk).
 int hc_commit(void* handle, int n, const int* slots, const int* tokens) {
   Core* core = (Core*)handle;
   for (int i = 0; i < n; ++i)
@@ -223,9 +225,10 @@ int hc_commit(void* handle, int n, const int* slots, const int* tokens) {
     const int slot = slots[i];
     core->length[slot] += tokens[i];
     for (Group& group : core->groups) {
-      if (group.window <= 0) continue;
+      if (group.window == 0) continue;
       Table& table = group.tables[slot];
-      const long first_needed_key = (long)core->length[slot] - group.window + 1;
+      const long length = core->length[slot];
+      const long first_needed_key = group.window > 0 ? length - group.window + 1 : length - length % -(long)group.window;
       if (first_needed_key <= 0) continue;
       const int first_needed_page = (int)std::min<long>(first_needed_key / group.page_size, (long)table.pages.size());
       // the pages of the kept first keys are never passed: what is given back starts behind them

@@ -69,7 +69,7 @@ __device__ __forceinline__ void route_token(const RouteArgs& a, int token) {
     if (j >= held) break;
     const int e = lane + WAVE * j;
     score[j] = e < E ? row[e] : -INFINITY;
-    choice[j] = e < E ? a.correction[e] : 0.f;     // (asked for beside the logits)
+    choice[j] = (a.correction && e < E) ? a.correction[e] : 0.f;     // (asked for beside the logits)
     most = fmaxf(most, score[j]);
   }
   if (a.mode == 0) {
@@ -89,6 +89,16 @@ __device__ __forceinline__ void route_token(const RouteArgs& a, int token) {
       const int e = lane + WAVE * j;
       score[j] = score[j] / total;
       choice[j] = e < E ? score[j] + choice[j] : -INFINITY;
+    }
+  } else if (a.mode == 2) {
+    // every output on its own: s = sigmoid(z).  Without a correction the logits decide, whose order is that of the s
+#pragma unroll
+    for (int j = 0; j < PER_LANE; ++j) {
+      if (j >= held) break;
+      const int e = lane + WAVE * j;
+      const float logit = score[j];
+      score[j] = e < E ? 1.0f / (1.0f + expf(-logit)) : 0.f;
+      choice[j] = e < E ? (a.correction ? score[j] + choice[j] : logit) : -INFINITY;
     }
   } else {
     // the logits with their bias are what is chosen by and what is weighted
@@ -147,7 +157,7 @@ __device__ __forceinline__ void route_token(const RouteArgs& a, int token) {
         own = score[j];
       }
     float best_score = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, own), best_id & (WAVE - 1)));
-    if (a.mode != 0) {
+    if (a.mode == 1) {
       if (k == 0) first_picked = best_score;
       best_score = expf(best_score - first_picked);
     }
@@ -180,10 +190,10 @@ __global__ void __launch_bounds__(256) moe_route_kernel(RouteArgs a) {
 }
 
 static int check_route(const RouteArgs& a) {
-  if (!a.logits || !a.correction || !a.chosen || !a.weights || a.T <= 0 || a.E <= 0 || a.top <= 0 || a.top > a.E || a.ld < a.E + (a.gate ? 1 : 0))
+  if (!a.logits || !a.chosen || !a.weights || a.T <= 0 || a.E <= 0 || a.top <= 0 || a.top > a.E || a.ld < a.E + (a.gate ? 1 : 0))
     return ERR_BAD_ARGUMENT;
   if (a.E > MOE_MAX_EXPERTS) return ERR_UNSUPPORTED_SIZE;
-  if (a.mode != 0 && a.mode != 1) return ERR_BAD_ARGUMENT;
+  if (a.mode < 0 || a.mode > 2) return ERR_BAD_ARGUMENT;
   if (a.mode == 1 && (!a.renormalize || a.groups != 0)) return ERR_BAD_ARGUMENT;
   if (a.groups < 0 || (a.groups > 0 && (a.E % a.groups != 0 || a.kept_groups <= 0 || a.kept_groups > a.groups ||
                                         a.kept_groups * (a.E / a.groups) < a.top)))
@@ -195,6 +205,7 @@ static int check_route(const RouteArgs& a) {
 // or without `renormalize` score * scale.  groups > 0 (mode 0): E / groups neighbouring experts form a group, its score
 // is its largest score + correction, and only experts of the `kept_groups` best groups can be chosen.
 // mode 1: choice by logit + correction (a bias), weights the softmax over the chosen (logit + correction) * scale.
+// mode 2: as mode 0 with the sigmoid of each logit in place of the softmax.  correction may be null (nothing is added).
 extern "C" int mi_moe_route(const float* logits, long ld, int T, int E, int top, const float* correction, float scale,
                             float eps, int mode, int renormalize, int groups, int kept_groups, int* chosen, float* weights,
                             float* gate, hipStream_t stream) {
@@ -215,6 +226,8 @@ struct PlanArgs {
   int* place;
   int* tile_expert;
   int* ranks;
+  const float* weights;             // with place_weight: the choices' weights, laid beside the places (padding gets 0)
+  float* place_weight;
 };
 
 // By one workgroup; a choice of E or beyond is an identity expert and gets the place -1.
@@ -222,7 +235,10 @@ __device__ __forceinline__ void plan_rows(const PlanArgs& a, int* counts, int* o
   const int tid = threadIdx.x;
   const int threads = blockDim.x;
   for (int e = tid; e < a.E; e += threads) counts[e] = 0;
-  for (int i = tid; i < a.capacity; i += threads) a.source[i] = -1;
+  for (int i = tid; i < a.capacity; i += threads) {
+    a.source[i] = -1;
+    if (a.place_weight) a.place_weight[i] = 0.f;
+  }
   for (int t = tid; t < a.capacity / a.pad; t += threads) a.tile_expert[t] = -1;
   __syncthreads();
   for (int i = tid; i < a.entries; i += threads) {
@@ -261,6 +277,7 @@ __device__ __forceinline__ void plan_rows(const PlanArgs& a, int* counts, int* o
     const int at = offsets[expert] + a.ranks[i];
     a.source[at] = i / a.top;
     a.place[i] = at;
+    if (a.place_weight) a.place_weight[at] = a.weights[i];
   }
 }
 
@@ -271,6 +288,7 @@ __global__ void __launch_bounds__(1024) moe_plan_kernel(PlanArgs a) {
 }
 
 static int check_plan(const PlanArgs& a) {
+  if (a.place_weight && !a.weights) return ERR_BAD_ARGUMENT;
   if (!a.chosen || !a.source || !a.place || !a.tile_expert || !a.ranks || a.entries <= 0 || a.top <= 0 || a.E <= 0 || a.pad <= 0 ||
       a.capacity % a.pad != 0 || a.capacity < a.entries + a.E * (a.pad - 1))
     return ERR_BAD_ARGUMENT;
@@ -278,8 +296,8 @@ static int check_plan(const PlanArgs& a) {
 }
 
 extern "C" int mi_moe_plan(const int* chosen, int entries, int top, int E, int pad, int capacity, int* source, int* place,
-                           int* tile_expert, int* ranks, hipStream_t stream) {
-  const PlanArgs a = {chosen, entries, top, E, pad, capacity, source, place, tile_expert, ranks};
+                           int* tile_expert, int* ranks, const float* weights, float* place_weight, hipStream_t stream) {
+  const PlanArgs a = {chosen, entries, top, E, pad, capacity, source, place, tile_expert, ranks, weights, place_weight};
   const int code = check_plan(a);
   if (code) return code;
   moe_plan_kernel<<<1, 1024, 0, stream>>>(a);
@@ -304,9 +322,9 @@ __global__ void __launch_bounds__(1024) moe_route_plan_kernel(RouteArgs route, P
 extern "C" int mi_moe_route_plan(const float* logits, long ld, int T, int E, int top, const float* correction, float scale,
                                  float eps, int mode, int renormalize, int groups, int kept_groups, int* chosen,
                                  float* weights, float* gate, int experts, int pad, int capacity, int* source, int* place,
-                                 int* tile_expert, int* ranks, hipStream_t stream) {
+                                 int* tile_expert, int* ranks, float* place_weight, hipStream_t stream) {
   const RouteArgs route = {logits, ld, T, E, top, correction, scale, eps, mode, renormalize, groups, kept_groups, chosen, weights, gate};
-  const PlanArgs plan = {chosen, T * top, top, experts, pad, capacity, source, place, tile_expert, ranks};
+  const PlanArgs plan = {chosen, T * top, top, experts, pad, capacity, source, place, tile_expert, ranks, weights, place_weight};
   int code = check_route(route);
   if (!code) code = check_plan(plan);
   if (code) return code;
@@ -329,7 +347,8 @@ template <typename T, typename TO, bool VEC, bool GLU, int MT, int PAIRS>
 __global__ void __launch_bounds__(TILE_THREADS)
 moe_expert_gemm_kernel(const T* __restrict__ x, long ldx, int x_rows, const T* __restrict__ W, long expert_stride, long ldw,
                        int N, int K, const int* __restrict__ source, const int* __restrict__ tile_expert, int gather,
-                       float limit, float alpha, float offset, int squared_relu, TO* __restrict__ out, long ldo) {
+                       float limit, float alpha, float offset, int squared_relu,
+                       const float* __restrict__ row_scale, TO* __restrict__ out, long ldo) {
   __shared__ float red[TILE_WAVES][256];
   const int tile = blockIdx.y;
   const int expert = tile_expert[tile];
@@ -361,9 +380,11 @@ moe_expert_gemm_kernel(const T* __restrict__ x, long ldx, int x_rows, const T* _
   for (int p = 0; p < PAIRS; ++p)
 #pragma unroll
     for (int mt = 0; mt < MT; ++mt) {
-      float value = tile_reduce(acc[p][mt], red);
+      const int place = (tile * MT + mt) * 16 + (l % 16);
+      const float scale = row_scale ? row_scale[place] : 1.0f;
+      float value = tile_reduce(acc[p][mt], red) * scale;
       if (GLU) {
-        const float up = tile_reduce(acc[NT - PAIRS + p][mt], red);
+        const float up = tile_reduce(acc[NT - PAIRS + p][mt], red) * scale;
         const float g = fminf(value, limit);
         const float u = fminf(fmaxf(up, -limit), limit);
         value = g / (1.0f + expf(-alpha * g)) * (u + offset);
@@ -372,7 +393,6 @@ moe_expert_gemm_kernel(const T* __restrict__ x, long ldx, int x_rows, const T* _
         value *= value;
       }
       const long n = n0 + 16 * p + 4 * (l / 16) + tid / 64;
-      const int place = (tile * MT + mt) * 16 + (l % 16);
       if (n < width) out[(long)place * ldo + n] = from_float<TO>(source[place] >= 0 ? value : 0.f);
     }
 }
@@ -391,8 +411,8 @@ template <typename T, typename TO, bool GLU>
 __global__ void __launch_bounds__(TILE_THREADS)
 moe_expert_gemm_wide_kernel(const T* __restrict__ x, long ldx, int x_rows, const T* __restrict__ W, long expert_stride,
                             long ldw, int N, int K, const int* __restrict__ source, const int* __restrict__ tile_expert,
-                            int gather, float limit, float alpha, float offset, int squared_relu, TO* __restrict__ out,
-                            long ldo) {
+                            int gather, float limit, float alpha, float offset, int squared_relu,
+                            const float* __restrict__ row_scale, TO* __restrict__ out, long ldo) {
   typedef typename TileTraits<T>::Piece Piece;
   constexpr int CHUNK = TileTraits<T>::CHUNK;
   constexpr int PIECE = TileTraits<T>::PIECE;
@@ -464,20 +484,21 @@ moe_expert_gemm_wide_kernel(const T* __restrict__ x, long ldx, int x_rows, const
   for (int mt = 0; mt < 4; ++mt) {
     const int place = tile * ROWS + 16 * mt + r;
     const bool live = source[place] >= 0;
+    const float scale = row_scale ? row_scale[place] : 1.0f;
     TO* row = out + (long)place * ldo;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       if (GLU) {
         const long n = n0 + 16 * wave + 4 * q + i;
-        const float g = fminf(acc[0][mt][i], limit);
-        const float u = fminf(fmaxf(acc[1][mt][i], -limit), limit);
+        const float g = fminf(acc[0][mt][i] * scale, limit);
+        const float u = fminf(fmaxf(acc[1][mt][i] * scale, -limit), limit);
         const float value = g / (1.0f + expf(-alpha * g)) * (u + offset);
         if (n < width) row[n] = from_float<TO>(live ? value : 0.f);
       } else {
 #pragma unroll
         for (int nt = 0; nt < 2; ++nt) {
           const long n = n0 + 32 * wave + 16 * nt + 4 * q + i;
-          float value = acc[nt][mt][i];
+          float value = acc[nt][mt][i] * scale;
           if (squared_relu) {
             value = fmaxf(value, 0.f);
             value *= value;
@@ -496,8 +517,8 @@ template <typename T, typename TO, bool GLU>
 __global__ void __launch_bounds__(TILE_THREADS)
 moe_expert_gemm_widest_kernel(const T* __restrict__ x, long ldx, int x_rows, const T* __restrict__ W, long expert_stride,
                               long ldw, int N, int K, const int* __restrict__ source, const int* __restrict__ tile_expert,
-                              int gather, float limit, float alpha, float offset, int squared_relu, TO* __restrict__ out,
-                              long ldo) {
+                              int gather, float limit, float alpha, float offset, int squared_relu,
+                              const float* __restrict__ row_scale, TO* __restrict__ out, long ldo) {
   typedef typename TileTraits<T>::Piece Piece;
   constexpr int CHUNK = TileTraits<T>::CHUNK;
   constexpr int PIECE = TileTraits<T>::PIECE;
@@ -577,6 +598,7 @@ moe_expert_gemm_widest_kernel(const T* __restrict__ x, long ldx, int x_rows, con
   for (int mt = 0; mt < 4; ++mt) {
     const int place = tile * ROWS + 64 * wm + 16 * mt + r;
     const bool live = source[place] >= 0;
+    const float scale = row_scale ? row_scale[place] : 1.0f;
     TO* row = out + (long)place * ldo;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -584,8 +606,8 @@ moe_expert_gemm_widest_kernel(const T* __restrict__ x, long ldx, int x_rows, con
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
           const long n = n0 + 32 * wn + 16 * h + 4 * q + i;
-          const float g = fminf(acc[h][mt][i], limit);
-          const float u = fminf(fmaxf(acc[2 + h][mt][i], -limit), limit);
+          const float g = fminf(acc[h][mt][i] * scale, limit);
+          const float u = fminf(fmaxf(acc[2 + h][mt][i] * scale, -limit), limit);
           const float value = g / (1.0f + expf(-alpha * g)) * (u + offset);
           if (n < width) row[n] = from_float<TO>(live ? value : 0.f);
         }
@@ -593,7 +615,7 @@ moe_expert_gemm_widest_kernel(const T* __restrict__ x, long ldx, int x_rows, con
 #pragma unroll
         for (int nt = 0; nt < 4; ++nt) {
           const long n = n0 + 64 * wn + 16 * nt + 4 * q + i;
-          float value = acc[nt][mt][i];
+          float value = acc[nt][mt][i] * scale;
           if (squared_relu) {
             value = fmaxf(value, 0.f);
             value *= value;
@@ -608,31 +630,32 @@ moe_expert_gemm_widest_kernel(const T* __restrict__ x, long ldx, int x_rows, con
 template <typename T, typename TO>
 static void launch_expert_gemm(const T* x, long ldx, int x_rows, const T* W, long expert_stride, long ldw, int N, int K,
                                const int* source, const int* tile_expert, int tiles, int pad, int gather, int activation,
-                               float limit, float alpha, float offset, TO* out, long ldo, hipStream_t stream) {
+                               float limit, float alpha, float offset, const float* row_scale, TO* out, long ldo,
+                               hipStream_t stream) {
   const int glu = activation == 1;
   const int squared_relu = activation == 2;
   constexpr int PIECE = TileTraits<T>::PIECE;
   const bool vec = K % PIECE == 0 && ldx % PIECE == 0 && ldw % PIECE == 0 && expert_stride % PIECE == 0 &&
                    ((unsigned long long)x % 16) == 0 && ((unsigned long long)W % 16) == 0;
   const int width = glu ? N / 2 : N;
-#define EXPERT_LAUNCH(VEC_, GLU_, MT_, PAIRS_)                                                                           moe_expert_gemm_kernel<T, TO, VEC_, GLU_, MT_, PAIRS_>                                                                    <<<dim3((unsigned)((width + 16 * PAIRS_ - 1) / (16 * PAIRS_)), (unsigned)tiles), TILE_THREADS, 0, stream>>>(               x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, out, ldo)
+#define EXPERT_LAUNCH(VEC_, GLU_, MT_, PAIRS_)                                                                           moe_expert_gemm_kernel<T, TO, VEC_, GLU_, MT_, PAIRS_>                                                                    <<<dim3((unsigned)((width + 16 * PAIRS_ - 1) / (16 * PAIRS_)), (unsigned)tiles), TILE_THREADS, 0, stream>>>(               x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, row_scale, out, ldo)
 #define EXPERT_SHAPE(MT_, PAIRS_GLU_, PAIRS_PLAIN_)                                                                      do {                                                                                                                    if (vec && glu) EXPERT_LAUNCH(true, true, MT_, PAIRS_GLU_);                                                            else if (vec) EXPERT_LAUNCH(true, false, MT_, PAIRS_PLAIN_);                                                           else if (glu) EXPERT_LAUNCH(false, true, MT_, PAIRS_GLU_);                                                             else EXPERT_LAUNCH(false, false, MT_, PAIRS_PLAIN_);                                                                 } while (0)
   if (pad == 128) {      // (only plans of rows and matrices in whole pieces are made so wide)
     const dim3 grid((unsigned)((width + (glu ? 64 : 128) - 1) / (glu ? 64 : 128)), (unsigned)tiles);
     if (glu)
       moe_expert_gemm_widest_kernel<T, TO, true><<<grid, TILE_THREADS, 0, stream>>>(
-          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, out, ldo);
+          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, row_scale, out, ldo);
     else
       moe_expert_gemm_widest_kernel<T, TO, false><<<grid, TILE_THREADS, 0, stream>>>(
-          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, out, ldo);
+          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, row_scale, out, ldo);
   } else if (pad == 64 && vec) {
     const dim3 grid((unsigned)((width + (glu ? 64 : 128) - 1) / (glu ? 64 : 128)), (unsigned)tiles);
     if (glu)
       moe_expert_gemm_wide_kernel<T, TO, true><<<grid, TILE_THREADS, 0, stream>>>(
-          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, out, ldo);
+          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, row_scale, out, ldo);
     else
       moe_expert_gemm_wide_kernel<T, TO, false><<<grid, TILE_THREADS, 0, stream>>>(
-          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, out, ldo);
+          x, ldx, x_rows, W, expert_stride, ldw, N, K, source, tile_expert, gather, limit, alpha, offset, squared_relu, row_scale, out, ldo);
   } else if (pad == 64) {
     EXPERT_SHAPE(4, 2, 4);
   } else {
@@ -644,8 +667,10 @@ static void launch_expert_gemm(const T* x, long ldx, int x_rows, const T* W, lon
 
 extern "C" int mi_moe_expert_gemm(const void* x, int dtype, long ldx, int x_rows, const void* W, long expert_stride,
                                   long ldw, int N, int K, const int* source, const int* tile_expert, int tiles, int pad,
-                                  int gather, int activation, float limit, float alpha, float offset, void* out,
-                                  int out_dtype, long ldo, hipStream_t stream) {
+                                  int gather, int activation, float limit, float alpha, float offset,
+                                  const float* row_scale, void* out, int out_dtype, long ldo, hipStream_t stream) {
+  // row_scale (or null): a number for every place that multiplies its row before the product (as the products are linear
+  // in the row, the sums before the activation)
   // activation: 0 none, 1 the clamped gated one (the matrix holds gate rows then up rows), 2 max(z, 0)^2
   const int glu = activation == 1;
   if (activation < 0 || activation > 2) return ERR_BAD_ARGUMENT;
@@ -661,13 +686,13 @@ extern "C" int mi_moe_expert_gemm(const void* x, int dtype, long ldx, int x_rows
   }
   if (dtype == DT_F32 && out_dtype == DT_F32)
     launch_expert_gemm<float, float>((const float*)x, ldx, x_rows, (const float*)W, expert_stride, ldw, N, K, source,
-                                     tile_expert, tiles, pad, gather, activation, limit, alpha, offset, (float*)out, ldo, stream);
+                                     tile_expert, tiles, pad, gather, activation, limit, alpha, offset, row_scale, (float*)out, ldo, stream);
   else if (dtype == DT_BF16 && out_dtype == DT_BF16)
     launch_expert_gemm<bf16_t, bf16_t>((const bf16_t*)x, ldx, x_rows, (const bf16_t*)W, expert_stride, ldw, N, K, source,
-                                       tile_expert, tiles, pad, gather, activation, limit, alpha, offset, (bf16_t*)out, ldo, stream);
+                                       tile_expert, tiles, pad, gather, activation, limit, alpha, offset, row_scale, (bf16_t*)out, ldo, stream);
   else if (dtype == DT_BF16 && out_dtype == DT_F32)
     launch_expert_gemm<bf16_t, float>((const bf16_t*)x, ldx, x_rows, (const bf16_t*)W, expert_stride, ldw, N, K, source,
-                                      tile_expert, tiles, pad, gather, activation, limit, alpha, offset, (float*)out, ldo, stream);
+                                      tile_expert, tiles, pad, gather, activation, limit, alpha, offset, row_scale, (float*)out, ldo, stream);
   else
     return ERR_BAD_ARGUMENT;
   RETURN_IF_LAUNCH_FAILED();
@@ -676,7 +701,7 @@ extern "C" int mi_moe_expert_gemm(const void* x, int dtype, long ldx, int x_rows
 
 // ---------------------------------------------------------------- a token's weighted sum
 // total[t, i] = sum over the choices k of weights[t, k] * (down[place[t, k], i], or x[t, i] where the place is negative),
-// + (gate[t], or one) * shared[t, i].  Without a tail out = total.  With one the sum goes on into the residual stream in
+// + (gate[t], or one) * shared[t, i]; weights null: every choice counts once.  Without a tail out = total.  With one the sum goes on into the residual stream in
 // the same launch: h += tanh(post_alpha total) * post_w + post_b, and (next_w not null) the new rows through the next
 // tanh norm, next_out = tanh(next_alpha h) * next_w + next_b.  A thread takes PIECE neighbouring features of a token.
 struct CombineTail {
@@ -744,7 +769,7 @@ moe_combine_kernel(const float* __restrict__ down, long ld, const int* __restric
     for (int u = 0; u < 4; ++u) {
       const int k = min(k0 + u, top - 1);
       at[u] = place[token * top + k];
-      weight[u] = k0 + u < top ? weights[token * top + k] : 0.f;
+      weight[u] = k0 + u < top ? (weights ? weights[token * top + k] : 1.0f) : 0.f;
     }
 #pragma unroll
     for (int u = 0; u < 4; ++u) piece_of<PIECE>(down + (long)max(at[u], 0) * ld + i, value[u]);
@@ -788,7 +813,7 @@ extern "C" int mi_moe_combine(const float* down, long ld, const int* place, cons
                               const float* gate, float* out, int T, int d, float* h, const float* post_w,
                               const float* post_b, float post_alpha, const float* next_w, const float* next_b,
                               float next_alpha, void* next_out, hipStream_t stream) {
-  if (!down || !place || !weights || T <= 0 || d <= 0 || top <= 0 || ld < d || (shared && shared_ld < d) || (x && x_ld < d))
+  if (!down || !place || T <= 0 || d <= 0 || top <= 0 || ld < d || (shared && shared_ld < d) || (x && x_ld < d))
     return ERR_BAD_ARGUMENT;
   if (h ? (!post_w || !post_b || (next_w && (!next_b || !next_out))) : !out) return ERR_BAD_ARGUMENT;
   const CombineTail tail = {h, post_w, post_b, next_w, next_b, post_alpha, next_alpha, next_out};

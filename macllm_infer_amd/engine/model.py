@@ -37,6 +37,8 @@ class DecoderModel:
         out = [Expect(f"{spec.embedding_name}.weight", ((spec.vocab_size, spec.hidden_size),), init="embedding")]
         if spec.bigram is not None:
             out.append(Expect(f"{spec.bigram_name}.weight", ((spec.bigram.buckets + 1, spec.hidden_size),), init="embedding"))
+        if spec.embedding_norm is not None:
+            out += part_class(spec.embedding_norm).expected_tensors(spec.embedding_norm, spec.embedding_norm_name, spec.hidden_size)
         for name, rows in spec.injected_vectors:
             out.append(Expect(name, ((rows, spec.hidden_size),), init="bias"))
         for name in spec.injected_mixes:
@@ -98,6 +100,10 @@ class DecoderModel:
         if build.dtype == torch.float32:
             table = table.to(torch.float32)
         self.embedding = table.contiguous().to(build.device)
+        self.embedding_norm = None
+        if spec.embedding_norm is not None:              # (weight, eps) of the norm the stream starts behind
+            norm = part_class(spec.embedding_norm)(spec.embedding_norm, spec.embedding_norm_name, tensors, build)
+            self.embedding_norm = norm.rms_prologue()
         self.bigram = None
         if spec.bigram is not None:
             table = tensors[f"{spec.bigram_name}.weight"]
@@ -168,7 +174,7 @@ class DecoderModel:
         spec = self.spec
         h = torch.empty((step.num_tokens, spec.hidden_size), dtype=torch.float32, device=self.build.device)
         if self.bigram is None:
-            ops.embed(step.token_ids, self.embedding, spec.embedding_multiplier, h)
+            ops.embed(step.token_ids, self.embedding, spec.embedding_multiplier, h, norm=self.embedding_norm)
         else:
             ops.embed_bigram(step.token_ids, self.embedding, spec.embedding_multiplier, self.bigram, spec.bigram.buckets,
                              spec.bigram.mul_prev, spec.bigram.mul_cur, step.positions, step.lane_of_token,

@@ -31,12 +31,13 @@ class KernelError(RuntimeError):
 _SIGNATURES = {
     "common": {
         "mi_embed": [_c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_int, _c_ptr],
+        "mi_embed_rmsnorm": [_c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_float, _c_ptr, _c_int, _c_int, _c_ptr],
         "mi_feed_tokens": [_c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
         "mi_add_rmsnorm": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_int,
                            _c_int, _c_float, _c_float, _c_ptr],
         "mi_add_partials_rmsnorm": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_int, _c_int,
                                     _c_int, _c_ptr],
-        "mi_swiglu": [_c_ptr, _c_int, _c_long, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+        "mi_swiglu": [_c_ptr, _c_int, _c_long, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_ptr],
         "mi_cast_rows": [_c_ptr, _c_ptr, _c_int, _c_long, _c_int, _c_int, _c_ptr],
         "mi_scale_to_f32": [_c_ptr, _c_int, _c_float, _c_ptr, _c_long, _c_ptr],
         "mi_tanh_softcap": [_c_ptr, _c_float, _c_long, _c_ptr],
@@ -51,6 +52,8 @@ _SIGNATURES = {
         "mi_add_layernorm": [_c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_float, _c_ptr,
                              _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_int, _c_int,
                              _c_ptr],
+        "mi_add_normed_rmsnorm": [_c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_float,
+                                  _c_ptr, _c_float, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
         "mi_add_tanhnorm": [_c_ptr, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_float, _c_ptr, _c_int, _c_float, _c_ptr,
                             _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
         "mi_clamped_glu": [_c_ptr, _c_int, _c_long, _c_ptr, _c_long, _c_int, _c_int, _c_float, _c_float, _c_float, _c_ptr],
@@ -73,16 +76,17 @@ _SIGNATURES = {
     "moe": {
         "mi_moe_route": [_c_ptr, _c_long, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_float, _c_int, _c_int, _c_int, _c_int,
                          _c_ptr, _c_ptr, _c_ptr, _c_ptr],
-        "mi_moe_plan": [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr],
+        "mi_moe_plan": [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                        _c_ptr],
         "mi_moe_expert_gemm": [_c_ptr, _c_int, _c_long, _c_int, _c_ptr, _c_long, _c_long, _c_int, _c_int, _c_ptr, _c_ptr,
-                               _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_ptr, _c_int, _c_long,
-                               _c_ptr],
+                               _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_ptr, _c_ptr, _c_int,
+                               _c_long, _c_ptr],
         "mi_moe_combine": [_c_ptr, _c_long, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_long, _c_ptr, _c_int, _c_long, _c_ptr,
                            _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_ptr,
                            _c_ptr],
         "mi_moe_route_plan": [_c_ptr, _c_long, _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_float, _c_int, _c_int, _c_int,
                               _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
-                              _c_ptr],
+                              _c_ptr, _c_ptr],
     },
     "linear_state": {
         "mi_linear_state_scan": [_c_ptr, _c_int, _c_long, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr,
@@ -111,14 +115,14 @@ _SIGNATURES = {
                                _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
                                _c_float, _c_int, _c_int,
                                _c_ptr, _c_long, _c_ptr, _c_long, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
-                               _c_ptr],
+                               _c_ptr, _c_long, _c_ptr],
         "mi_attention_prepare": [_c_ptr, _c_int, _c_long, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr,
                                  _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_float, _c_int, _c_ptr, _c_ptr, _c_float,
-                                 _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_long, _c_int, _c_ptr],
+                                 _c_float, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_long, _c_int, _c_ptr],
         "mi_paged_attention_workspace": [_c_int, _c_int, _c_int, _c_int],
         "mi_prefill_attention": [_c_ptr, _c_long, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_long, _c_int, _c_ptr,
                                  _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int, _c_int, _c_ptr, _c_long,
-                                 _c_ptr, _c_ptr, _c_int, _c_ptr],
+                                 _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_long, _c_ptr],
         "mi_prefill_attention_forms": [_c_ptr, _c_long, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_long, _c_int,
                                        _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int, _c_int, _c_ptr,
                                        _c_long, _c_int, _c_ptr, _c_ptr, _c_ptr],
@@ -127,7 +131,13 @@ _SIGNATURES = {
                                 _c_ptr, _c_long, _c_ptr],
         "mi_decode_attention_forms": [_c_ptr, _c_long, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_long,
                                       _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int, _c_int, _c_int, _c_ptr,
-                                      _c_ptr, _c_ptr, _c_long, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr],
+                                      _c_ptr, _c_ptr, _c_long, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr,
+                                      _c_long, _c_ptr],
+    },
+    "attention_widths": {
+        "mi_prefill_attention_padded": [_c_ptr, _c_long, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_long, _c_int,
+                                        _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int, _c_int, _c_ptr,
+                                        _c_long, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_long, _c_ptr],
     },
     "mamba2": {
         "mi_conv1d_silu": [_c_ptr, _c_int, _c_long, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
@@ -155,7 +165,7 @@ _SIGNATURES = {
         "mi_fused_gemm": [_c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_long, _c_ptr,
                           _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_long, _c_int, _c_float, _c_int, _c_int, _c_int,
                           _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_int, _c_int, _c_float, _c_int,
-                          _c_ptr],
+                          _c_float, _c_float, _c_float, _c_ptr],
         "mi_fused_gemm_residual": [_c_ptr, _c_long, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_long,
                                    _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
         "mi_fused_gemm_tanh": [_c_ptr, _c_long, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_float,
@@ -260,14 +270,38 @@ def _row_major(tensor: torch.Tensor, name: str) -> int:
     return tensor.stride(0) if tensor.shape[0] > 1 else max(tensor.stride(0), tensor.shape[1])
 
 
+def _span(window: Optional[int], chunk: Optional[int], name: str) -> int:
+    """What the attention kernels take for the keys a query sees: a window's size, the negated size of chunks, or 0."""
+    _need(not (window and chunk), f"{name}: a window or chunks, not both")
+    _need((window or 0) >= 0 and (chunk or 0) >= 0, f"{name}: windows and chunks have positive sizes")
+    return -int(chunk) if chunk else int(window or 0)
+
+
+def _gate_rows(gate: Optional[torch.Tensor], out: torch.Tensor, name: str) -> int:
+    """The row stride of a gate on the heads' outputs (0 without one)."""
+    if gate is None:
+        return 0
+    _need(gate.shape == out.shape and gate.dtype == out.dtype, f"{name}: the gate must have the output's shape and dtype")
+    return _row_major(gate, "gate")
+
+
 # --------------------------------------------------------------------------- common
-def embed(token_ids: torch.Tensor, table: torch.Tensor, multiplier: float, out: torch.Tensor) -> None:
-    """out[t] = table[token_ids[t]] * multiplier, out float32 [T, d]."""
+def embed(token_ids: torch.Tensor, table: torch.Tensor, multiplier: float, out: torch.Tensor,
+          norm: Optional[tuple] = None) -> None:
+    """out[t] = table[token_ids[t]] * multiplier, out float32 [T, d]; with ``norm`` (weight float32 [d], eps) each row e
+    becomes e / sqrt(mean(e^2) + eps) * weight."""
     _i32(token_ids, "token_ids")
     T, d = out.shape
     _need(token_ids.numel() == T and table.dim() == 2 and table.shape[1] == d and table.is_contiguous(),
           "embed: shapes do not match")
     _need(out.dtype == torch.float32 and out.is_contiguous(), "embed: out must be contiguous float32")
+    if norm is not None:
+        weight, eps = norm
+        _need(weight.dtype == torch.float32 and weight.numel() == d and weight.is_contiguous() and weight.is_cuda and eps > 0,
+              "embed: the norm's weight must be float32 [d] on the GPU and its eps positive")
+        _check(_fn("common", "mi_embed_rmsnorm")(_p(token_ids), _p(table), _dt(table), float(multiplier), _p(weight),
+                                                 float(eps), _p(out), T, d, _stream()), "embed")
+        return
     _check(_fn("common", "mi_embed")(_p(token_ids), _p(table), _dt(table), float(multiplier), _p(out), T, d,
                                      _stream()), "embed")
 
@@ -338,13 +372,20 @@ def add_partials_rmsnorm(h: torch.Tensor, partial: torch.Tensor, weight: torch.T
         None, T, T, d, _stream()), "add_partials_rmsnorm", f"(d={d}, S={partial.shape[0]})")
 
 
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
 
 
-def swiglu(gate_up: torch.Tensor, out: torch.Tensor, tile: int = 0, activation: str = "silu") -> None:
+def _clamp_numbers(activation: str, clamp, name: str) -> tuple:
+    """(limit, alpha, up_offset) of the activation "clamped", which ``clamp`` brings; zeros for the others."""
+    _need((activation == "clamped") == (clamp is not None), f"{name}: the clamped activation and its numbers come together")
+    return (float(clamp.limit), float(clamp.alpha), float(clamp.up_offset)) if clamp is not None else (0.0, 0.0, 0.0)
+
+
+def swiglu(gate_up: torch.Tensor, out: torch.Tensor, tile: int = 0, activation: str = "silu", clamp=None) -> None:
     """out[t, i] = act(g[t, i]) * u[t, i] with a row of ``gate_up`` holding [g | u] (``tile`` 0) or
     g and u interleaved in tiles of ``tile`` columns: [g[0:tile] | u[0:tile] | g[tile:2 tile] | ...]; act is SiLU
-    or ("gelu_tanh") 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))."""
+    or ("gelu_tanh") 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))).  Activation "clamped" (``clamp``: limit, alpha,
+    up_offset): out = g * sigmoid(alpha g) * (u + up_offset) with g = min(g, limit), u = clamp(u, -limit, limit)."""
     _need(activation in GATE_ACTIVATIONS, f"swiglu: the activation {activation!r} is not known")
     ld = _row_major(gate_up, "gate_up")
     T, two_i = gate_up.shape
@@ -352,7 +393,8 @@ def swiglu(gate_up: torch.Tensor, out: torch.Tensor, tile: int = 0, activation: 
           "swiglu: out must be contiguous [T, I] of the input's dtype")
     _need(tile >= 0 and (tile == 0 or (two_i // 2) % tile == 0), "swiglu: the tile must divide the width")
     _check(_fn("common", "mi_swiglu")(_p(gate_up), _dt(gate_up), ld, _p(out), T, two_i // 2, int(tile),
-                                      GATE_ACTIVATIONS[activation], _stream()), "swiglu")
+                                      GATE_ACTIVATIONS[activation], *_clamp_numbers(activation, clamp, "swiglu"),
+                                      _stream()), "swiglu")
 
 
 def cast_rows(source: torch.Tensor, out: torch.Tensor) -> None:
@@ -527,6 +569,42 @@ def add_layernorm(h: torch.Tensor, branches: Sequence[tuple], vector: Optional[t
     _check(_fn("common", "mi_add_layernorm")(
         _p(h), *flat, _p(vector), _p(weight), _p(bias), float(eps), _p(post[0]), _p(post[1]), float(post[2]), _p(out),
         _dt(out) if out is not None else DT_F32, _p(rows), n_rows, d, _stream()), "add_layernorm", f"(d={d})")
+
+
+def add_normed_rmsnorm(h: torch.Tensor, branches: Sequence[tuple], branch_norm: tuple, weight: Optional[torch.Tensor],
+                       eps: float, out: Optional[torch.Tensor], rows: Optional[torch.Tensor] = None) -> None:
+    """s = sum of factor * branch over ``branches`` [(tensor [T, d], factor)] (one to three);
+    h += s / sqrt(mean(s^2) + branch eps) * branch weight with ``branch_norm`` (weight, eps) (float32, in place);
+    out = h / sqrt(mean(h^2) + eps) * weight.  With ``rows`` only those rows are read, ``out[i]`` gets row ``rows[i]`` and
+    ``h`` is left as it is.  Without ``out`` nothing is normed behind the add, and ``weight`` may be None."""
+    _need(h.dtype == torch.float32 and h.dim() == 2 and h.is_contiguous() and h.is_cuda,
+          "add_normed_rmsnorm: h must be contiguous float32 [T, d]")
+    T, d = h.shape
+    _need(1 <= len(branches) <= 3, "add_normed_rmsnorm: one to three branches")
+    for tensor, _ in branches:
+        _need(tensor.shape == h.shape and tensor.is_contiguous(), "add_normed_rmsnorm: branches must be contiguous [T, d]")
+    for name, one in [("the branches' weight", branch_norm[0])] + ([("weight", weight)] if out is not None else []):
+        _need(one is not None and one.dtype == torch.float32 and one.numel() == d and one.is_contiguous() and one.is_cuda,
+              f"add_normed_rmsnorm: {name} must be float32 [d] on the GPU")
+    n_rows = T
+    if rows is not None:
+        _i32(rows, "rows")
+        n_rows = rows.numel()
+        _need(out is not None, "add_normed_rmsnorm: a gather needs somewhere to put its rows")
+    if out is not None:
+        _need(out.shape == (n_rows, d) and out.is_contiguous(), "add_normed_rmsnorm: out must be contiguous [rows, d]")
+    if n_rows == 0:
+        return
+    flat = []
+    for index in range(3):
+        if index < len(branches):
+            tensor, factor = branches[index]
+            flat += [_p(tensor), _dt(tensor), float(factor)]
+        else:
+            flat += [None, DT_F32, 0.0]
+    _check(_fn("common", "mi_add_normed_rmsnorm")(
+        _p(h), *flat, _p(branch_norm[0]), float(branch_norm[1]), _p(weight) if out is not None else None, float(eps), _p(out),
+        _dt(out) if out is not None else DT_F32, _p(rows), n_rows, d, _stream()), "add_normed_rmsnorm", f"(d={d})")
 
 
 def add_tanhnorm(h: torch.Tensor, branches: Sequence[tuple], weight: Optional[torch.Tensor], bias: Optional[torch.Tensor],
@@ -783,17 +861,20 @@ def moe_tile_rows(tokens: int, top_k: int, num_experts: int, whole_pieces: bool 
     return MOE_WIDE_TILE_ROWS if tokens * top_k >= MOE_WIDE_TILE_ROWS * num_experts else MOE_TILE_ROWS
 
 
+ROUTINGS = {"softmax_then_top": 0, "top_then_softmax": 1, "sigmoid_then_top": 2}
+
+
 def _route_arguments(logits, num_experts, top_k, correction, shared_gate, routing, groups, kept_groups, name):
     """Checks of a routing call; (row length, tokens, chosen, weights, gate)."""
     _need(groups == 0 or (num_experts % groups == 0 and 0 < kept_groups <= groups
-                          and kept_groups * (num_experts // groups) >= top_k and routing == "softmax_then_top"),
+                          and kept_groups * (num_experts // groups) >= top_k and routing != "top_then_softmax"),
           f"{name}: the groups do not fit the experts")
-    _need(routing in ("softmax_then_top", "top_then_softmax"), f"{name}: routing {routing!r} is not known")
+    _need(routing in ROUTINGS, f"{name}: routing {routing!r} is not known")
     ld = _row_major(logits, "logits")
     T = logits.shape[0]
     _need(logits.dtype == torch.float32 and logits.shape[1] >= num_experts + (1 if shared_gate else 0),
           f"{name}: float32 logits of every expert")
-    _need(correction.dtype == torch.float32 and correction.numel() == num_experts and correction.is_cuda,
+    _need(correction is None or (correction.dtype == torch.float32 and correction.numel() == num_experts and correction.is_cuda),
           f"{name}: the correction must be float32 [experts] on the GPU")
     _need(0 < top_k <= num_experts, f"{name}: a token uses at least one and at most all experts")
     chosen = torch.empty((T, top_k), dtype=torch.int32, device=logits.device)
@@ -802,7 +883,7 @@ def _route_arguments(logits, num_experts, top_k, correction, shared_gate, routin
     return ld, T, chosen, weights, gate
 
 
-def moe_route(logits: torch.Tensor, num_experts: int, top_k: int, correction: torch.Tensor, scale: float, eps: float,
+def moe_route(logits: torch.Tensor, num_experts: int, top_k: int, correction: Optional[torch.Tensor], scale: float, eps: float,
               shared_gate: bool, routing: str = "softmax_then_top", renormalize: bool = True, groups: int = 0,
               kept_groups: int = 0):
     """From float32 router logits [T, >= num_experts (+ 1)]: s = softmax over the experts; the ``top_k`` largest of
@@ -810,13 +891,14 @@ def moe_route(logits: torch.Tensor, num_experts: int, top_k: int, correction: to
     [T, top_k]) s / (sum of the chosen s + eps) * scale; with ``shared_gate`` also sigmoid of column
     ``num_experts`` (float32 [T]), else None.  ``routing`` "top_then_softmax": the ``top_k`` largest of
     logits + correction (the correction is then a bias of the logits) are chosen, and their weights are the softmax
-    over these alone, times scale.  ``renormalize`` False: the weights are s * scale.  ``groups``: the experts form that
+    over these alone, times scale.  ``routing`` "sigmoid_then_top": s is the sigmoid of each logit.  ``renormalize`` False:
+    the weights are s * scale.  ``correction`` None: nothing is added.  ``groups``: the experts form that
     many equal groups of neighbours, and only those of the ``kept_groups`` groups with the largest s + correction in
     them can be chosen.  (``num_experts`` counts every output of the router, experts without matrices included.)"""
     ld, T, chosen, weights, gate = _route_arguments(logits, num_experts, top_k, correction, shared_gate, routing, groups,
                                                     kept_groups, "moe_route")
     _check(_fn("moe", "mi_moe_route")(_p(logits), ld, T, num_experts, top_k, _p(correction), float(scale), float(eps),
-                                      0 if routing == "softmax_then_top" else 1, 1 if renormalize else 0, int(groups),
+                                      ROUTINGS[routing], 1 if renormalize else 0, int(groups),
                                       int(kept_groups), _p(chosen), _p(weights), _p(gate), _stream()), "moe_route",
            f"(experts={num_experts})")
     return chosen, weights, gate
@@ -827,9 +909,10 @@ class MoePlan:
     stands at a place (-1: padding), ``place`` int32 [T * top_k] = where a token's choice stands, ``tile_expert``
     int32 [capacity / pad] = the expert of every tile of ``pad`` places (-1: an unused tile).  A choice of
     ``num_experts`` or beyond (an expert without matrices) stands nowhere: its place is -1.  Every expert's rows
-    start a tile; ``capacity`` depends on the number of tokens alone."""
+    start a tile; ``capacity`` depends on the number of tokens alone.  ``place_weight`` (float32 [capacity], if asked for):
+    the weight of the choice that stands at a place (padding: 0)."""
 
-    def __init__(self, tokens: int, top_k: int, num_experts: int, pad: Optional[int], device):
+    def __init__(self, tokens: int, top_k: int, num_experts: int, pad: Optional[int], device, weighted: bool = False):
         pad = moe_tile_rows(tokens, top_k, num_experts) if pad is None else int(pad)
         self.pad, self.tokens, self.top_k = pad, tokens, top_k
         self.capacity = -(-(tokens * top_k + num_experts * (pad - 1)) // pad) * pad
@@ -837,15 +920,21 @@ class MoePlan:
         self.place = torch.empty((tokens * top_k,), dtype=torch.int32, device=device)
         self.tile_expert = torch.empty((self.capacity // pad,), dtype=torch.int32, device=device)
         self.ranks = torch.empty((tokens * top_k,), dtype=torch.int32, device=device)
+        self.place_weight = torch.empty((self.capacity,), dtype=torch.float32, device=device) if weighted else None
 
 
-def moe_plan(chosen: torch.Tensor, num_experts: int, pad: Optional[int] = None) -> MoePlan:
-    """The plan of the choices ``chosen`` int32 [T, top_k]."""
+def moe_plan(chosen: torch.Tensor, num_experts: int, pad: Optional[int] = None,
+             weights: Optional[torch.Tensor] = None) -> MoePlan:
+    """The plan of the choices ``chosen`` int32 [T, top_k]; with ``weights`` float32 [T, top_k] their weights lie beside
+    the places."""
     _i32(chosen, "chosen")
     tokens, top_k = chosen.shape
-    plan = MoePlan(tokens, top_k, num_experts, pad, chosen.device)
+    _need(weights is None or (weights.dtype == torch.float32 and weights.shape == chosen.shape and weights.is_contiguous()
+                              and weights.is_cuda), "moe_plan: the weights must be float32 [T, top_k] on the GPU")
+    plan = MoePlan(tokens, top_k, num_experts, pad, chosen.device, weights is not None)
     _check(_fn("moe", "mi_moe_plan")(_p(chosen), tokens * top_k, top_k, num_experts, plan.pad, plan.capacity, _p(plan.source),
-                                     _p(plan.place), _p(plan.tile_expert), _p(plan.ranks), _stream()),
+                                     _p(plan.place), _p(plan.tile_expert), _p(plan.ranks), _p(weights),
+                                     _p(plan.place_weight), _stream()),
            "moe_plan", f"(experts={num_experts})")
     return plan
 
@@ -853,30 +942,35 @@ def moe_plan(chosen: torch.Tensor, num_experts: int, pad: Optional[int] = None) 
 ROUTE_PLAN_TOKENS = 64      # steps of up to this many tokens are routed and grouped in one launch
 
 
-def moe_route_plan(logits: torch.Tensor, num_experts: int, top_k: int, correction: torch.Tensor, scale: float, eps: float,
+def moe_route_plan(logits: torch.Tensor, num_experts: int, top_k: int, correction: Optional[torch.Tensor], scale: float, eps: float,
                    shared_gate: bool, *, experts_with_matrices: int, pad: Optional[int] = None,
-                   routing: str = "softmax_then_top", renormalize: bool = True, groups: int = 0, kept_groups: int = 0):
-    """``moe_route`` and ``moe_plan`` of a step of up to ROUTE_PLAN_TOKENS tokens in one launch: (chosen, weights, gate,
-    plan).  ``experts_with_matrices``: the experts that the plan groups rows for (the router's first outputs)."""
+                   routing: str = "softmax_then_top", renormalize: bool = True, groups: int = 0, kept_groups: int = 0,
+                   place_weights: bool = False):
+    """``moe_route`` and ``moe_plan`` (``place_weights``: with the weights beside the places) of a step of up to
+    ROUTE_PLAN_TOKENS tokens in one launch: (chosen, weights, gate, plan).  ``experts_with_matrices``: the experts that the plan groups rows for (the router's first outputs)."""
     ld, T, chosen, weights, gate = _route_arguments(logits, num_experts, top_k, correction, shared_gate, routing, groups,
                                                     kept_groups, "moe_route_plan")
     _need(T <= ROUTE_PLAN_TOKENS and 0 < experts_with_matrices <= num_experts, "moe_route_plan: the step or its experts do not fit")
-    plan = MoePlan(T, top_k, experts_with_matrices, pad, logits.device)
+    plan = MoePlan(T, top_k, experts_with_matrices, pad, logits.device, place_weights)
     _check(_fn("moe", "mi_moe_route_plan")(
         _p(logits), ld, T, num_experts, top_k, _p(correction), float(scale), float(eps),
-        0 if routing == "softmax_then_top" else 1, 1 if renormalize else 0, int(groups), int(kept_groups), _p(chosen),
+        ROUTINGS[routing], 1 if renormalize else 0, int(groups), int(kept_groups), _p(chosen),
         _p(weights), _p(gate), experts_with_matrices, plan.pad, plan.capacity, _p(plan.source), _p(plan.place),
-        _p(plan.tile_expert), _p(plan.ranks), _stream()), "moe_route_plan", f"(experts={num_experts})")
+        _p(plan.tile_expert), _p(plan.ranks), _p(plan.place_weight), _stream()), "moe_route_plan", f"(experts={num_experts})")
     return chosen, weights, gate, plan
 
 
 def moe_expert_gemm(x: torch.Tensor, plan: MoePlan, weight: torch.Tensor, out: torch.Tensor, gather: bool, glu,
-                    squared_relu: bool = False) -> None:
+                    squared_relu: bool = False, row_scale: Optional[torch.Tensor] = None) -> None:
     """The grouped product of a plan's rows with their experts' matrices ``weight`` [experts, N, K]: the row at a
     place is ``x[source[place]]`` (``gather``) or ``x[place]``; out[place] = weight[expert] . row, or with ``glu``
     (limit, alpha, up_offset; N = 2 I, gate rows then up rows) the clamped gated activation of the two halves,
     [capacity, I]; or with ``squared_relu`` max(weight[expert] . row, 0)^2.  Float32 sums on the matrix cores;
-    float32 operands give a true 32-bit product."""
+    float32 operands give a true 32-bit product.  ``row_scale`` float32 [capacity]: a number that multiplies a place's row
+    before the product (applied, in float32, to the sums before the activation)."""
+    _need(row_scale is None or (row_scale.dtype == torch.float32 and row_scale.numel() == plan.capacity
+                                and row_scale.is_contiguous() and row_scale.is_cuda),
+          "moe_expert_gemm: row_scale must be float32 [capacity] on the GPU")
     _need(not (squared_relu and glu is not None), "moe_expert_gemm: one activation")
     ldx = _row_major(x, "x")
     ldo = _row_major(out, "out")
@@ -890,7 +984,7 @@ def moe_expert_gemm(x: torch.Tensor, plan: MoePlan, weight: torch.Tensor, out: t
         _p(x), _dt(x), ldx, x.shape[0], _p(weight), N * K, K, N, K, _p(plan.source), _p(plan.tile_expert),
         plan.tile_expert.numel(), plan.pad, 1 if gather else 0, 1 if glu is not None else (2 if squared_relu else 0),
         float(glu.limit) if glu is not None else 0.0, float(glu.alpha) if glu is not None else 0.0,
-        float(glu.up_offset) if glu is not None else 0.0, _p(out), _dt(out), ldo, _stream()),
+        float(glu.up_offset) if glu is not None else 0.0, _p(row_scale), _p(out), _dt(out), ldo, _stream()),
         "moe_expert_gemm", f"(N={N}, K={K})")
 
 
@@ -910,19 +1004,20 @@ def _tanh_tail(tail: tuple, T: int, d: int, dtype, name: str) -> list:
     return [_p(h), _p(post[0]), _p(post[1]), float(post[2]), _p(after[0]), _p(after[1]), float(after[2]), _p(rows)]
 
 
-def moe_combine(down: torch.Tensor, plan: MoePlan, weights: torch.Tensor, shared_rows: Optional[torch.Tensor],
+def moe_combine(down: torch.Tensor, plan: MoePlan, weights: Optional[torch.Tensor], shared_rows: Optional[torch.Tensor],
                 shared_gate: Optional[torch.Tensor], out: Optional[torch.Tensor], own_rows: Optional[torch.Tensor] = None,
                 tail: Optional[tuple] = None) -> None:
     """out[t] = sum over the token's choices k, in their order, of weights[t, k] * down[place[t, k]]
     (+ shared_gate[t] * shared_rows[t], or shared_rows[t] as they are without a gate), float32.  ``own_rows`` [T, d]:
     what a choice without a place (an expert that returns its input) contributes in place of a row of ``down``.
+    ``weights`` None: every choice counts once.
     ``tail`` (h, post norm, next norm or None, next rows or None; in place of ``out``): the sum goes on into the residual
     stream, h += tanh(alpha sum) * weight + bias, and the new rows through the next tanh norm into the next rows."""
     _need((out is None) != (tail is None), "moe_combine: the sum goes to out or into the stream")
     T, d = plan.tokens, down.shape[1]
     ld = _row_major(down, "down")
-    _need(down.dtype == torch.float32 and weights.dtype == torch.float32 and weights.shape == (T, plan.top_k)
-          and weights.is_contiguous(), "moe_combine: shapes do not fit the plan")
+    _need(down.dtype == torch.float32 and (weights is None or (weights.dtype == torch.float32
+          and weights.shape == (T, plan.top_k) and weights.is_contiguous())), "moe_combine: shapes do not fit the plan")
     _need(out is None or (out.dtype == torch.float32 and out.is_contiguous() and out.shape == (T, d)),
           "moe_combine: out must be contiguous float32 [T, d]")
     shared_ld = 0
@@ -1208,7 +1303,8 @@ def paged_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim
                     log_bias: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None,
                     value_dim: Optional[int] = None, head_scales: Optional[torch.Tensor] = None,
                     score_bias: Optional[torch.Tensor] = None, sigmoid: bool = False, keep_first: int = 0,
-                    fixed_sink: Optional[float] = None) -> None:
+                    fixed_sink: Optional[float] = None, chunk: Optional[int] = None,
+                    gate: Optional[torch.Tensor] = None) -> None:
     """Causal attention of every token over its request's cached keys (its own included).
 
     ``q`` [T, >= Hq*dh] (rotated); ``block_tables`` [lanes, max_pages] page ids by logical
@@ -1225,7 +1321,10 @@ def paged_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim
     [Hq]): every head's scores are multiplied by its number (after ``scale``).  ``sigmoid``: a visible key weighs
     sigmoid(score + ``score_bias[head]``) (float32 [Hq] or None) on its own and nothing is normalized.
     ``keep_first`` (with a window): keys at positions below it stay visible behind the window.  ``fixed_sink``: a
-    sink of this score for every head, in place of ``sinks``."""
+    sink of this score for every head, in place of ``sinks``.  ``chunk`` (in place of a window): a query sees the keys
+    of its own chunk of that many positions, counted from the sequence's start.  ``gate`` (``out``'s shape and dtype):
+    what is written is multiplied by sigmoid(gate)."""
+    span_code = _span(window, chunk, "paged_attention")
     _need(keep_first >= 0 and (keep_first == 0 or window), "paged_attention: first keys are kept behind a window")
     _need(fixed_sink is None or (sinks is None and not sigmoid), "paged_attention: one sink, in a softmax")
     q_ld = _row_major(q, "q")
@@ -1266,10 +1365,11 @@ def paged_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim
     _check(_fn("attention", "mi_paged_attention")(
         _p(q), _dt(q), q_ld, T, num_heads, num_kv_heads, head_dim, value_dim, _p(k_cache), _p(v_cache), page_stride,
         page_size, _p(block_tables), block_tables.shape[1], _p(lane_of_token), _p(positions), float(scale),
-        int(window or 0), int(keep_first), _p(slopes), _p(log_bias), _p(sinks),
+        span_code, int(keep_first), _p(slopes), _p(log_bias), _p(sinks),
         float(fixed_sink or 0.0), 0 if fixed_sink is None else 1, span, _p(partial), partial.numel(), _p(out), out_ld,
         _p(query_tiles) if tiles else None, tiles, int(tile_tokens) if tiles else 0, _p(cu_seqlens) if tiles else None,
-        _p(head_scales), _p(score_bias), 1 if sigmoid else 0, _stream()), "paged_attention", f"(head_dim={head_dim})")
+        _p(head_scales), _p(score_bias), 1 if sigmoid else 0, _p(gate), _gate_rows(gate, out, "paged_attention"),
+        _stream()), "paged_attention", f"(head_dim={head_dim})")
 
 
 def attention_prepare(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
@@ -1280,7 +1380,7 @@ def attention_prepare(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head
                       norm_eps: float = 0.0, value_inv_freq: Optional[torch.Tensor] = None,
                       interleaved: bool = False, turn_scale: float = 1.0, head_norm: Optional[str] = None,
                       q_head_weight: Optional[torch.Tensor] = None, k_head_weight: Optional[torch.Tensor] = None,
-                      head_eps: float = 0.0) -> None:
+                      head_eps: float = 0.0, temperature: Optional[tuple] = None) -> None:
     """A token's projected row made ready for attention, one launch: ``qkv`` [T, >= Hq*dh + Hkv*dh (+ Hkv*dv)]
     holds q heads, k heads and (unless ``values_from_keys``) v heads.
 
@@ -1296,7 +1396,12 @@ def attention_prepare(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head
       with ``value_inv_freq`` (float32 [dv / 2]) they are turned by the position over all their dims (half-split
       pairs); they go to the token's (transposed) cache cell.
 
+    ``temperature`` (coef, every): the queries are multiplied by 1 + coef * ln(floor((position + 1) / every) + 1) at the
+    end.  ``num_kv_heads`` 0 (without ``slot_mapping``): a row of queries alone, whose keys another layer has cached.
     Norms, angles and rotations are float32.  Without ``slot_mapping`` nothing is stored."""
+    _need(num_kv_heads > 0 or (slot_mapping is None and q_norm is None and not values_from_keys),
+          "attention_prepare: a row of queries alone stores nothing")
+    _need(temperature is None or int(temperature[1]) > 0, "attention_prepare: the temperature's step must be positive")
     ld = _row_major(qkv, "qkv")
     T = qkv.shape[0]
     value_dim = int(value_dim)
@@ -1336,36 +1441,48 @@ def attention_prepare(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head
         _p(positions), _p(inv_freq), int(rotary_dim) if inv_freq is not None else 0, 1 if interleaved else 0,
         float(turn_scale), _p(q_norm), _p(k_norm), float(norm_eps),
         {None: 0, "before_rotation": 1, "after_rotation": 2}[head_norm], _p(q_head_weight), _p(k_head_weight),
-        float(head_eps), _p(value_inv_freq), _p(slot_mapping), _p(k_cache) if slot_mapping is not None else None,
+        float(head_eps), float(temperature[0]) if temperature is not None else 0.0,
+        int(temperature[1]) if temperature is not None else 0, _p(value_inv_freq), _p(slot_mapping), _p(k_cache) if slot_mapping is not None else None,
         _p(v_cache) if slot_mapping is not None else None, page_stride, page_size, _stream()), "attention_prepare")
 
 
-def prefill_attention_supported(dtype, num_heads: int, num_kv_heads: int, head_dim: int, page_size: int) -> bool:
-    """Whether the matrix-core attention kernel covers this geometry."""
-    return (dtype == torch.bfloat16 and head_dim in (64, 128) and page_size % 4 == 0
-            and num_heads // num_kv_heads <= 64)
+def prefill_attention_supported(dtype, num_heads: int, num_kv_heads: int, head_dim: int, page_size: int,
+                                value_dim: Optional[int] = None) -> bool:
+    """Whether the matrix-core attention kernel covers this geometry.  Without ``value_dim`` the question is whether it
+    does so at its own widths (heads of 64 or 128, values as wide); with it, padding counts too."""
+    if not (dtype == torch.bfloat16 and page_size % 4 == 0 and num_heads // num_kv_heads <= 64):
+        return False
+    if head_dim in (64, 128) and value_dim in (None, head_dim):
+        return True
+    return value_dim is not None and head_dim % 8 == 0 and head_dim <= 128 and value_dim % 4 == 0 and value_dim <= 128
 
 
 def prefill_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, k_cache: torch.Tensor,
                       v_cache: torch.Tensor, block_tables: torch.Tensor, query_tiles: torch.Tensor,
                       cu_seqlens: torch.Tensor, start_pos: torch.Tensor, scale: float, window: Optional[int],
                       out: torch.Tensor, max_seq_len: int = 0, log_bias: Optional[torch.Tensor] = None,
-                      sinks: Optional[torch.Tensor] = None, keep_first: int = 0) -> None:
+                      sinks: Optional[torch.Tensor] = None, keep_first: int = 0, chunk: Optional[int] = None,
+                      slopes: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                      value_dim: Optional[int] = None) -> None:
     """``paged_attention`` on the matrix cores for bfloat16 (flash-style, online softmax in
     float32).  ``query_tiles`` [tiles, 2]: (lane, first token row) of runs of up to 64 tokens of
     one lane; the keys and values of the step's own tokens must be in the cache already.
     ``max_seq_len``: an upper bound of the step's longest context if known (it picks how many heads share
-    a key fragment, never the result).  ``keep_first`` (with a window): keys at positions below it stay visible."""
+    a key fragment, never the result).  ``keep_first`` (with a window): keys at positions below it stay visible.
+    ``chunk``, ``slopes``, ``gate``, ``value_dim``: as for ``paged_attention``.  Heads of 64 or 128 with values as wide
+    take the kernel of their width; any other width up to 128 the one that pads to the next of its own."""
     _need(keep_first >= 0 and (keep_first == 0 or window), "prefill_attention: first keys are kept behind a window")
+    span_code = _span(window, chunk, "prefill_attention")
+    value_dim = head_dim if value_dim is None else int(value_dim)
     q_ld = _row_major(q, "q")
     out_ld = _row_major(out, "out")
     T = q.shape[0]
     _need(q.dtype == torch.bfloat16 and out.dtype == torch.bfloat16, "prefill_attention: bfloat16 only")
-    _need(q.shape[1] >= num_heads * head_dim and out.shape == (T, num_heads * head_dim) and q_ld % 8 == 0
+    _need(q.shape[1] >= num_heads * head_dim and out.shape == (T, num_heads * value_dim) and q_ld % 8 == 0
           and q.data_ptr() % 16 == 0 and out_ld % 4 == 0 and out.data_ptr() % 8 == 0,
           "prefill_attention: q/out shapes or alignment do not fit")
-    page_stride, page_size = _cache_view(k_cache, v_cache, num_kv_heads, head_dim, q.dtype)
-    _need(prefill_attention_supported(q.dtype, num_heads, num_kv_heads, head_dim, page_size),
+    page_stride, page_size = _cache_view(k_cache, v_cache, num_kv_heads, head_dim, q.dtype, value_dim)
+    _need(prefill_attention_supported(q.dtype, num_heads, num_kv_heads, head_dim, page_size, value_dim),
           "prefill_attention: geometry not covered; use paged_attention")
     for name, tensor in (("block_tables", block_tables), ("query_tiles", query_tiles), ("cu_seqlens", cu_seqlens),
                          ("start_pos", start_pos)):
@@ -1378,11 +1495,17 @@ def prefill_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
           "prefill_attention: log_bias must be float32 [Hq, 2] on the GPU")
     _need(sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == num_heads and sinks.is_contiguous()
                             and sinks.is_cuda), "prefill_attention: sinks must be float32 [Hq] on the GPU")
-    _check(_fn("attention", "mi_prefill_attention")(
-        _p(q), q_ld, num_heads, num_kv_heads, head_dim, _p(k_cache), _p(v_cache), page_stride, page_size,
-        _p(block_tables), block_tables.shape[1], _p(query_tiles), query_tiles.shape[0], _p(cu_seqlens),
-        _p(start_pos), float(scale), int(window or 0), int(max_seq_len or 0), _p(out), out_ld, _p(log_bias),
-        _p(sinks), int(keep_first), _stream()), "prefill_attention")
+    _need(slopes is None or (slopes.dtype == torch.float32 and slopes.numel() == num_heads and slopes.is_contiguous()
+                             and slopes.is_cuda and log_bias is None),
+          "prefill_attention: slopes must be float32 [Hq] on the GPU, and stand in place of log_bias")
+    gate_ld = _gate_rows(gate, out, "prefill_attention")
+    _need(gate is None or (gate_ld % 4 == 0 and gate.data_ptr() % 8 == 0), "prefill_attention: the gate's rows lie in pieces of four")
+    own_width = head_dim in (64, 128) and value_dim == head_dim
+    _check(_fn(*(("attention", "mi_prefill_attention") if own_width else ("attention_widths", "mi_prefill_attention_padded")))(
+        _p(q), q_ld, num_heads, num_kv_heads, head_dim, *(() if own_width else (value_dim,)), _p(k_cache), _p(v_cache),
+        page_stride, page_size, _p(block_tables), block_tables.shape[1], _p(query_tiles), query_tiles.shape[0],
+        _p(cu_seqlens), _p(start_pos), float(scale), span_code, int(max_seq_len or 0), _p(out), out_ld, _p(log_bias),
+        _p(sinks), int(keep_first), _p(slopes), _p(gate), gate_ld, _stream()), "prefill_attention")
 
 
 PREFILL_VALUE_WIDTH_MOST = 256      # the widest values the matrix-core kernel computes with
@@ -1439,7 +1562,7 @@ DECODE_KEEP_FIRST_MOST = 512        # DEC_MAX_SPLIT in attention.hip: the kept f
 def decode_attention_supported(dtype, num_heads: int, num_kv_heads: int, head_dim: int, page_size: int,
                                value_dim: Optional[int] = None, keep_first: int = 0) -> bool:
     """Whether the split-context kernel for single-token queries covers this geometry."""
-    return (dtype == torch.bfloat16 and head_dim in (64, 128) and num_heads // num_kv_heads <= 8
+    return (dtype == torch.bfloat16 and head_dim % 8 == 0 and head_dim <= 128 and num_heads // num_kv_heads <= 8
             and page_size % 8 == 0 and page_size <= 512 and (value_dim is None or 0 < value_dim <= 256)
             and keep_first <= DECODE_KEEP_FIRST_MOST)
 
@@ -1449,11 +1572,16 @@ def decode_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_di
                      positions: torch.Tensor, scale: float, window: Optional[int], max_seq_len: int,
                      out: torch.Tensor, value_dim: Optional[int] = None, head_scales: Optional[torch.Tensor] = None,
                      score_bias: Optional[torch.Tensor] = None, sigmoid: bool = False, keep_first: int = 0,
-                     sinks: Optional[torch.Tensor] = None) -> None:
+                     sinks: Optional[torch.Tensor] = None, chunk: Optional[int] = None,
+                     slopes: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
     """``paged_attention`` for batches of single decoded tokens in bfloat16: the context of each
     request is split over many workgroups and the G query heads of a kv head share its K/V
     loads.  ``max_seq_len``: an upper bound of the longest context in the batch.  ``value_dim``,
-    ``head_scales``, ``score_bias``, ``sigmoid``, ``keep_first`` and ``sinks`` as in ``paged_attention``."""
+    ``head_scales``, ``score_bias``, ``sigmoid``, ``keep_first``, ``sinks``, ``chunk``, ``slopes`` and ``gate`` as in
+    ``paged_attention``."""
+    span_code = _span(window, chunk, "decode_attention")
+    _need(slopes is None or (slopes.dtype == torch.float32 and slopes.numel() == num_heads and slopes.is_contiguous()
+                             and slopes.is_cuda), "decode_attention: slopes must be float32 [Hq] on the GPU")
     _need(keep_first >= 0 and (keep_first == 0 or window), "decode_attention: first keys are kept behind a window")
     _need(sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == num_heads and sinks.is_contiguous()
                             and sinks.is_cuda and not sigmoid), "decode_attention: sinks must be float32 [Hq] on the GPU")
@@ -1476,7 +1604,8 @@ def decode_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_di
         _need(one is None or (one.dtype == torch.float32 and one.numel() == num_heads and one.is_contiguous()
                               and one.is_cuda), f"decode_attention: {name} must be float32 [Hq] on the GPU")
     _need(sigmoid or score_bias is None, "decode_attention: a bias per head is for sigmoid weights")
-    span = max_seq_len if not window else min(max_seq_len, window + page_size)
+    most_seen = window or chunk
+    span = max_seq_len if not most_seen else min(max_seq_len, most_seen + page_size)
     split_keys = 64
     while split_keys < 512 and span * T * num_kv_heads > 1024 * split_keys:
         split_keys *= 2
@@ -1487,9 +1616,10 @@ def decode_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_di
     partial_ml = torch.empty((T, num_heads, blocks, 2), dtype=torch.float32, device=q.device)
     _check(_fn("attention", "mi_decode_attention_forms")(
         _p(q), q_ld, T, num_heads, num_kv_heads, head_dim, value_dim, _p(k_cache), _p(v_cache), page_stride, page_size,
-        _p(block_tables), block_tables.shape[1], _p(lane_of_token), _p(positions), float(scale), int(window or 0),
-        split_keys, splits, _p(partial_o), _p(partial_ml), _p(out), out_ld, _p(head_scales), _p(score_bias),
-        1 if sigmoid else 0, int(keep_first), _p(sinks), _stream()), "decode_attention")
+        _p(block_tables), block_tables.shape[1], _p(lane_of_token), _p(positions), float(scale), span_code,
+        split_keys, splits, _p(partial_o), _p(partial_ml), _p(out), out_ld, _p(head_scales), _p(score_bias), _p(slopes),
+        1 if sigmoid else 0, int(keep_first), _p(sinks), _p(gate), _gate_rows(gate, out, "decode_attention"), _stream()),
+        "decode_attention")
 
 
 # --------------------------------------------------------------------------- mamba2
@@ -1826,14 +1956,14 @@ def fused_gemm(weight: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Te
                norm_weight: Optional[torch.Tensor] = None, eps: float = 0.0, epilogue: int = EPI_PLAIN,
                conv: Optional[dict] = None, feature_tiles: int = 1, fragments: Optional[torch.Tensor] = None,
                row_scale: Optional["RowScale"] = None, shared_rows: bool = False, row_tiles: int = 1,
-               gate_activation: str = "silu") -> None:
+               gate_activation: str = "silu", clamp=None) -> None:
     """out[M, N'] = epilogue(prologue . weight[N, K]^T + bias) for a small batch in bfloat16.
 
     Prologue: ``x`` [M, K] bfloat16, or ``h_in`` float32 [M, K] with up to two bfloat16 ``deltas``:
     the rows are summed (the sum goes to ``h_out``, a different tensor, if given), RMS-normed
     with ``norm_weight`` and ``eps``.  Epilogue PLAIN: bfloat16 or float32 ``out`` [M, N] times
     ``out_scale``.  SWIGLU: weight rows in tiles of 8 gate + 8 up rows, ``out`` [M, N/2] = act(gate) * up with
-    act = SiLU or, ``gate_activation`` "gelu_tanh", the tanh form of GELU.
+    act = SiLU or, ``gate_activation`` "gelu_tanh", the tanh form of GELU; "clamped" with ``clamp``: as for ``swiglu``.
     CONV: ``conv`` = {lo, hi, taps, weight [C, taps], bias, state [slots, taps-1, C], slot_ids}:
     rows lo..hi-1 go through the causal depthwise conv step of their channel with the request's
     tail (which is rolled) and SiLU.  ``feature_tiles`` (1, 2 or 4; more than one with ``x`` only): how many
@@ -1850,7 +1980,7 @@ def fused_gemm(weight: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Te
           "fused_gemm: weight must be contiguous bfloat16 [N, K]")
     _need(row_scale is None or x is not None, "fused_gemm: a row scale needs x")
     _need(gate_activation in GATE_ACTIVATIONS and (gate_activation == "silu" or epilogue == EPI_SWIGLU),
-          "fused_gemm: the gate's activation is silu or gelu_tanh, and belongs to the SWIGLU epilogue")
+          "fused_gemm: the gate's activation is silu, gelu_tanh or clamped, and belongs to the SWIGLU epilogue")
     _need(1 <= row_tiles <= 4 and (row_tiles == 1 or (x is not None and feature_tiles == 1 and not shared_rows)),
           "fused_gemm: row_tiles is 1 to 4, and more than 1 needs x, one feature tile and the skinny kernel")
     if row_scale is not None:
@@ -1903,7 +2033,7 @@ def fused_gemm(weight: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Te
         _p(slot_ids), -int(feature_tiles) if shared_rows else int(feature_tiles), int(fragments is not None),
         _p(row_scale.ssq) if row_scale is not None else None, row_scale.ssq.shape[0] if row_scale is not None else 0,
         int(row_scale.width) if row_scale is not None else 0, float(row_scale.eps) if row_scale is not None else 0.0,
-        int(row_tiles), _stream()), "fused_gemm", f"(M={M}, N={N}, K={K})")
+        int(row_tiles), *_clamp_numbers(gate_activation, clamp, "fused_gemm"), _stream()), "fused_gemm", f"(M={M}, N={N}, K={K})")
 
 
 @dataclass(frozen=True)

@@ -100,10 +100,11 @@ class NormedBranches:
     """Branch outputs whose weighted sum goes through a norm of its own before it joins the residual stream:
     x <- x + ((s - mean) / sqrt(variance + eps) * weight + bias) with s = sum of factor * rows over ``branches``
     [(rows [T, d], factor)], everything in float32; with ``alpha`` the norm is the one without statistics,
-    x <- x + (tanh(alpha s) * weight + bias)."""
+    x <- x + (tanh(alpha s) * weight + bias); with no ``bias`` it is an RMS norm, x <- x + s / sqrt(mean(s^2) + eps) *
+    weight."""
     branches: list
     weight: torch.Tensor
-    bias: torch.Tensor
+    bias: Optional[torch.Tensor] = None
     eps: float = 0.0
     alpha: Optional[float] = None
 

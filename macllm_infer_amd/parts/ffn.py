@@ -13,7 +13,8 @@ from .linear import Linear
 
 @register_part("swiglu")
 class SwiGLU(FeedForward):
-    """down(act(gate(x)) * up(x)), act = SiLU or the tanh form of GELU (``activation``); gate and up are one fused
+    """down(act(gate(x)) * up(x)), act = SiLU or the tanh form of GELU (``activation``), or down of the clamped gated
+    activation of gate(x) and up(x) (``clamp``); gate and up are one fused
     product (reference: src/decoder.rs:261-306).  ``gate_multiplier`` scales gate's output,
     ``down_multiplier`` down's output; both are folded into the weights.  When the width is a
     multiple of 8 the rows of the fused matrix are stored in tiles of 8 gate rows and 8 up rows
@@ -73,11 +74,11 @@ class SwiGLU(FeedForward):
             # epilogue (the weight rows already lie in its tiles of 8 gate and 8 up rows)
             activated = torch.empty((rows, self.spec.intermediate_size), dtype=x.dtype, device=x.device)
             ops.fused_gemm(self.gate_up.weight, self.gate_up.bias, activated, x=x, epilogue=ops.EPI_SWIGLU,
-                           gate_activation=self.spec.activation)
+                           gate_activation=self.spec.activation, clamp=self.spec.clamp)
             return activated
         gate_up = self.gate_up(x)
         activated = torch.empty((x.shape[0], self.spec.intermediate_size), dtype=gate_up.dtype, device=x.device)
-        ops.swiglu(gate_up, activated, self.tile, activation=self.spec.activation)
+        ops.swiglu(gate_up, activated, self.tile, activation=self.spec.activation, clamp=self.spec.clamp)
         return activated
 
 

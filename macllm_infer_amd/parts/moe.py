@@ -23,7 +23,9 @@ class RoutedExperts(FeedForward):
     An expert is down(act(gate(x), up(x))) with the clamped gated activation of ``ClampedGLUSpec`` and no biases, or
     (an activation that is not ``gated``) down(max(up(x), 0)^2) with no gate matrix.  With ``routing``
     "top_then_softmax" the router's logits get a bias, the largest are chosen and weighted by the softmax over the
-    chosen ones alone.  The router's logits are a float32 product (its weight is kept in 32 bits, with the shared expert's gate vector as
+    chosen ones alone; with "sigmoid_then_top" every score is the sigmoid of its own logit.  ``input_weighted``: a weight
+    multiplies its expert's input; it lies beside the row's place and multiplies the first product's sums, before the
+    activation.  The router's logits are a float32 product (its weight is kept in 32 bits, with the shared expert's gate vector as
     one more row); one kernel forms the softmax, adds the correction, picks the experts and their weights.  The
     tokens' rows are then grouped by expert on the device (no count travels to the host: the launch sizes depend on
     the number of tokens alone): each expert's rows fill whole tiles of the grouped products, gate/up with the
@@ -41,7 +43,7 @@ class RoutedExperts(FeedForward):
         out = [Expect(f"{prefix}.router.weight", ((spec.router_outputs, hidden_size),))]
         if spec.routing == "top_then_softmax":
             out.append(Expect(f"{prefix}.router.bias", ((spec.num_experts,),), init="bias"))
-        else:
+        elif spec.corrected:
             out.append(Expect(f"{prefix}.correction", ((spec.router_outputs,),), init="bias"))
         gated = getattr(spec.activation, "gated", True)
         for number in range(spec.num_experts):
@@ -96,8 +98,10 @@ class RoutedExperts(FeedForward):
                 self.shared_down = Linear([get("shared.down.weight")], [None], build)
         self.router = torch.cat(router).contiguous().to(build.device)
         # what is added to a token's scores before the choice: a correction of the softmax, or the logits' bias
-        added = "router.bias" if spec.routing == "top_then_softmax" else "correction"
-        self.correction = get(added).to(torch.float32).contiguous().to(build.device)
+        self.correction = None
+        if spec.corrected:
+            added = "router.bias" if spec.routing == "top_then_softmax" else "correction"
+            self.correction = get(added).to(torch.float32).contiguous().to(build.device)
         # rows and matrices in whole 16-byte pieces: the widest tiles of the grouped products take nothing else
         piece = 4 if keep == torch.float32 else 8
         self.whole_pieces = hidden % piece == 0 and inner % piece == 0
@@ -120,14 +124,17 @@ class RoutedExperts(FeedForward):
                   self.shared and spec.shared_gated)
         pad = ops.moe_tile_rows(tokens, spec.top_k, spec.num_experts, self.whole_pieces)
         if tokens <= ops.ROUTE_PLAN_TOKENS:
-            _, weights, gate, plan = ops.moe_route_plan(*choice, experts_with_matrices=spec.num_experts, pad=pad, **how)
+            _, weights, gate, plan = ops.moe_route_plan(*choice, experts_with_matrices=spec.num_experts, pad=pad,
+                                                         place_weights=spec.input_weighted, **how)
         else:
             chosen, weights, gate = ops.moe_route(*choice, **how)
-            plan = ops.moe_plan(chosen, spec.num_experts, pad)
+            plan = ops.moe_plan(chosen, spec.num_experts, pad, weights if spec.input_weighted else None)
+        if spec.input_weighted:                # the weights are in the rows: the sum of the experts' outputs is plain
+            weights = None
         rows = x if x.dtype == self.gate_up.dtype else x.to(self.gate_up.dtype)
         inner = torch.empty((plan.capacity, spec.expert_size), dtype=rows.dtype, device=x.device)
         ops.moe_expert_gemm(rows, plan, self.gate_up, inner, gather=True, glu=spec.activation if self.gated else None,
-                            squared_relu=not self.gated)
+                            squared_relu=not self.gated, row_scale=plan.place_weight if spec.input_weighted else None)
         down = torch.empty((plan.capacity, hidden), dtype=torch.float32, device=x.device)
         ops.moe_expert_gemm(inner, plan, self.down, down, gather=False, glu=None)
         shared_rows = self._shared_rows(x) if self.shared else None

@@ -40,6 +40,11 @@ def add_normed_branches(h: torch.Tensor, normed: NormedBranches, vector: Optiona
         second, factor = branches.pop(0)
         ops.stream_add(extra, second, factor, None)
         branches.insert(0, (extra, 1.0))
+    if normed.bias is None:
+        ops.add_normed_rmsnorm(h, branches, (normed.weight, normed.eps), None, 0.0, None)
+        if vector is not None:
+            ops.stream_add(h, None, 1.0, vector)
+        return
     if normed.alpha is not None:
         ops.add_tanhnorm(h, branches, None, None, 0.0, None, branch_norm=(normed.weight, normed.bias, normed.alpha))
         if vector is not None:
@@ -108,9 +113,23 @@ class RmsNorm(Part):
     def rms_prologue(self):
         return self.weight, self.eps
 
+    def behind_branches(self) -> dict:
+        """This norm as the one behind a layer's branches: what ``NormedBranches`` takes beside them."""
+        return dict(weight=self.weight, eps=self.eps)
+
     def forward(self, residual: Residual, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Add the pending branch outputs to the residual stream and return its normed rows
         (all of them, or only ``rows``; with ``rows`` the stream itself is left unchanged)."""
+        if (len(residual.pending) == 1 and isinstance(residual.pending[0], NormedBranches)
+                and residual.pending[0].bias is None and len(residual.pending[0].branches) <= LAYERNORM_BRANCHES):
+            # a branch through an RMS norm of its own, the add and this norm in one launch
+            normed = residual.pending[0]
+            count = residual.h.shape[0] if rows is None else rows.numel()
+            out = torch.empty((count, residual.h.shape[1]), dtype=self.build.dtype, device=residual.h.device)
+            ops.add_normed_rmsnorm(residual.h, normed.branches, (normed.weight, normed.eps), self.weight, self.eps, out, rows)
+            if rows is None:
+                residual.pending = []
+            return out
         if any(isinstance(branch, (RowVector, NormedBranches)) for branch in residual.pending):
             fold_weighted(residual, keep_weighted=True)
         if any(isinstance(branch, WeightedBranch) for branch in residual.pending):
@@ -210,7 +229,7 @@ class LayerNorm(Part):
         for branch in residual.pending:
             if isinstance(branch, NormedBranches):
                 # the one the kernel takes through its own norm on the way into the stream; others before it
-                if (normed is not None or rows is not None or branch.alpha is not None
+                if (normed is not None or rows is not None or branch.alpha is not None or branch.bias is None
                         or len(branch.branches) > LAYERNORM_BRANCHES):
                     add_normed_branches(residual.h, branch)
                 else:

@@ -151,6 +151,19 @@ class LogDistanceBias(PositionEncoding):
         return None
 
 
+@register_part("linear_distance")
+class LinearDistanceBias(PositionEncoding):
+    """No rotation of q and k: a key n positions behind the query loses slope[head] * n of its score, with the fixed
+    slopes of the spec (``LinearDistanceBiasSpec``)."""
+    graph_safe = True
+
+    def __init__(self, spec, head_dim: int, build: BuildContext):
+        self.score_slopes = torch.tensor(spec.slopes, dtype=torch.float64).to(torch.float32).to(build.device)
+
+    def pair_rotation(self):
+        return None, 0, False
+
+
 @register_part("rope_interleaved")
 class InterleavedRope(PositionEncoding):
     """Rotary encoding whose pairs are neighbouring dimensions: (u, v) = dimensions (2i, 2i + 1) at position p

@@ -46,17 +46,19 @@ def model_sizes(spec) -> dict:
                 values, mixed = part.num_kv_heads * part.value_width, part.num_heads * part.value_width
                 # values that are the keys as projected have no matrix of their own, but cells of their own in the cache
                 projected = 0 if getattr(part, "values_from_keys", False) else values
+                stored = entry.kv_from is None and getattr(part, "own_rows", True)
+                rows = q + (kv + projected if getattr(part, "own_rows", True) else 0) + (mixed if getattr(part, "out_gate", False) else 0)
                 if getattr(part, "projection_norm_eps", None) is not None:
                     total["in_weights"] += q + kv                          # the norms' weights over whole projections
-                total["in_weights"] += (q + kv + projected) * d
+                total["in_weights"] += rows * d
                 total["out_weights"] += d * mixed
-                total["kv_per_token"] += kv + values if entry.kv_from is None else 0
+                total["kv_per_token"] += kv + values if stored else 0
                 # x 2 T^2 flops (causal: half of 4 T^2); a window w keeps min(i + 1, w) keys for the query at i
                 total["attention"] += part.num_heads * (part.head_dim + part.value_width) / 2.0
                 total["windows"].append((part.num_heads * (part.head_dim + part.value_width) / 2.0,
-                                         (kv + values) if entry.kv_from is None else 0, part.window))
+                                         kv + values if stored else 0, Chunk(part.chunk) if getattr(part, "chunk", None) else part.window))
                 total["mixed"] += mixed
-                total["in_width"] += q + kv + projected
+                total["in_width"] += rows
                 if getattr(part, "conv_kernel", 0) > 1:                    # the tail of the projections' convolution
                     total["conv_tail"] += (part.conv_kernel - 1) * (q + kv + projected)
             elif part.kind == "gated_linear_attention":
@@ -138,8 +140,16 @@ def model_sizes(spec) -> dict:
     return total
 
 
+class Chunk(int):
+    """A chunk's size where a window's may stand."""
+
+
 def keys_seen(tokens: float, window) -> float:
-    """Sum over the queries 0 .. tokens-1 of one prompt of the keys each sees: min(i + 1, window)."""
+    """Sum over the queries 0 .. tokens-1 of one prompt of the keys each sees: min(i + 1, window), or with chunks
+    i mod chunk + 1."""
+    if isinstance(window, Chunk) and window < tokens:
+        whole, rest = tokens // window, tokens % window
+        return whole * window * (window + 1) / 2.0 + rest * (rest + 1) / 2.0
     if not window or window >= tokens:
         return tokens * (tokens + 1) / 2.0
     return window * (window + 1) / 2.0 + (tokens - window) * window
@@ -163,7 +173,8 @@ def decode_step_costs(spec, batch: int, context: float, element: int = 2) -> Dic
     unused = lambda top_k, experts: 2.0 * rows * (top_k - experts_touched(experts, top_k, rows))
     gate_up_flops = 2.0 * rows * s["gate_up"] + sum(unused(top_k, experts) * gate_up for experts, top_k, gate_up, _ in s["experts"])
     down_flops = 2.0 * rows * s["down"] + sum(unused(top_k, experts) * down for experts, top_k, _, down in s["experts"])
-    kept = lambda window: min(context, window) if window else context          # keys a query still sees
+    # keys a query still sees (with chunks: those of the chunk that the context ends in)
+    kept = lambda window: (context - 1) % window + 1 if isinstance(window, Chunk) else min(context, window) if window else context
     kv_read = sum(per_token * kept(window) for _, per_token, window in s["windows"])
     attention_flops = sum(4.0 * width * kept(window) for width, _, window in s["windows"])
     return {

@@ -16,8 +16,11 @@ def _f(t):
     return t.float()
 
 
-def embed(token_ids, table, multiplier, out):
-    out.copy_(_f(table)[token_ids.long()] * multiplier)
+def embed(token_ids, table, multiplier, out, norm=None):
+    rows = _f(table)[token_ids.long()] * multiplier
+    if norm is not None:
+        rows = rows / torch.sqrt(rows.pow(2).mean(-1, keepdim=True) + norm[1]) * norm[0]
+    out.copy_(rows)
 
 
 def feed_tokens(token_ids, source, dst, src):
@@ -47,7 +50,7 @@ def cast_rows(source, out):
 def attention_prepare(qkv, num_heads, num_kv_heads, head_dim, value_dim, positions, inv_freq, rotary_dim, slot_mapping,
                       k_cache, v_cache, *, values_from_keys=False, q_norm=None, k_norm=None, norm_eps=0.0,
                       value_inv_freq=None, interleaved=False, turn_scale=1.0, head_norm=None, q_head_weight=None,
-                      k_head_weight=None, head_eps=0.0):
+                      k_head_weight=None, head_eps=0.0, temperature=None):
     T = qkv.shape[0]
     q_cols, k_cols = num_heads * head_dim, num_kv_heads * head_dim
     q = _f(qkv[:, :q_cols]).clone()
@@ -88,6 +91,9 @@ def attention_prepare(qkv, num_heads, num_kv_heads, head_dim, value_dim, positio
         q, k = norm_heads(q, q_head_weight), norm_heads(k, k_head_weight)
     if value_inv_freq is not None:
         v = rotate(v, value_inv_freq, value_dim)
+    if temperature is not None:
+        coef, every = temperature
+        q = q * (1.0 + coef * torch.log(((positions.long() + 1) // every + 1).float()))[:, None, None]
     qkv[:, :q_cols] = q.reshape(T, q_cols).to(qkv.dtype)
     if slot_mapping is not None:
         page_size = k_cache.shape[2]
@@ -97,13 +103,16 @@ def attention_prepare(qkv, num_heads, num_kv_heads, head_dim, value_dim, positio
         v_cache[pages, :, :, offsets] = v.to(v_cache.dtype)
 
 
-def swiglu(gate_up, out, tile=0, activation="silu"):
+def swiglu(gate_up, out, tile=0, activation="silu", clamp=None):
     inner = gate_up.shape[1] // 2
     if tile:
         tiles = gate_up.reshape(gate_up.shape[0], inner // tile, 2, tile)
         gate, up = tiles[:, :, 0].reshape(-1, inner), tiles[:, :, 1].reshape(-1, inner)
     else:
         gate, up = gate_up[:, :inner], gate_up[:, inner:]
+    if activation == "clamped":
+        clamped_glu(torch.cat([gate, up], dim=1), clamp.limit, clamp.alpha, clamp.up_offset, out)
+        return
     if activation == "gelu_tanh":
         z = _f(gate)
         bent = 0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))
@@ -176,7 +185,7 @@ def rope_kv_store(qkv, num_heads, num_kv_heads, head_dim, positions, inv_freq, r
 def paged_attention(q, num_heads, num_kv_heads, head_dim, k_cache, v_cache, block_tables, lane_of_token,
                     positions, scale, window, out, max_seq_len=None, slopes=None, query_tiles=None, tile_tokens=0,
                     cu_seqlens=None, log_bias=None, sinks=None, value_dim=None, head_scales=None, score_bias=None,
-                    sigmoid=False, keep_first=0, fixed_sink=None):
+                    sigmoid=False, keep_first=0, fixed_sink=None, chunk=None, gate=None):
     """``max_seq_len`` sizes the kernel's launch and nothing else: not used here, and neither is the table of
     runs that picks the kernel for lanes of several tokens.  ``slopes``: a bias on the scores,
     ``-slopes[head] * (query position - key position)``; ``log_bias`` [Hq, 2] = (r1, r2): the scores lose
@@ -188,7 +197,7 @@ def paged_attention(q, num_heads, num_kv_heads, head_dim, k_cache, v_cache, bloc
     for token in range(T):
         lane = int(lane_of_token[token])
         position = int(positions[token])
-        first = 0 if not window else max(0, position - window + 1)
+        first = position - position % chunk if chunk else 0 if not window else max(0, position - window + 1)
         keys = torch.arange(first, position + 1)
         if keep_first and first > 0:
             keys = torch.cat([torch.arange(0, min(keep_first, first)), keys])
@@ -216,22 +225,24 @@ def paged_attention(q, num_heads, num_kv_heads, head_dim, k_cache, v_cache, bloc
             else:
                 weights = torch.softmax(scores, dim=0)
             out[token, head * value_dim:(head + 1) * value_dim] = (weights @ v[:, head // group, :]).to(out.dtype)
+    if gate is not None:
+        out.copy_((_f(out) * torch.sigmoid(_f(gate))).to(out.dtype))
 
 
 def decode_attention_supported(dtype, num_heads, num_kv_heads, head_dim, page_size, value_dim=None, keep_first=0):
     return False
 
 
-def prefill_attention_supported(dtype, num_heads, num_kv_heads, head_dim, page_size):
+def prefill_attention_supported(dtype, num_heads, num_kv_heads, head_dim, page_size, value_dim=None):
     return False
 
 
 def decode_attention(q, num_heads, num_kv_heads, head_dim, k_cache, v_cache, block_tables, lane_of_token, positions,
                      scale, window, max_seq_len, out, value_dim=None, head_scales=None, score_bias=None, sigmoid=False,
-                     keep_first=0, sinks=None):
+                     keep_first=0, sinks=None, chunk=None, slopes=None, gate=None):
     paged_attention(q, num_heads, num_kv_heads, head_dim, k_cache, v_cache, block_tables, lane_of_token, positions,
                     scale, window, out, value_dim=value_dim, head_scales=head_scales, score_bias=score_bias,
-                    sigmoid=sigmoid, keep_first=keep_first, sinks=sinks)
+                    sigmoid=sigmoid, keep_first=keep_first, sinks=sinks, chunk=chunk, slopes=slopes, gate=gate)
 
 
 def conv1d_silu(u, col_offset, width, weight, bias, conv_state, lane_of_token, cu_seqlens, slot_ids, out, activation=True):
@@ -441,6 +452,20 @@ def add_layernorm(h, branches, vector, weight, bias, eps, out, rows=None, branch
         out.copy_((centred / torch.sqrt(variance + eps) * weight + bias).to(out.dtype))
 
 
+def add_normed_rmsnorm(h, branches, branch_norm, weight, eps, out, rows=None):
+    summed = torch.zeros_like(h)
+    for tensor, factor in branches:
+        summed = summed + float(factor) * _f(tensor)
+    total = h + summed / torch.sqrt(summed.pow(2).mean(-1, keepdim=True) + branch_norm[1]) * branch_norm[0]
+    if rows is None:
+        h.copy_(total)
+        picked = total
+    else:
+        picked = total[rows.long()]
+    if out is not None:
+        out.copy_((picked / torch.sqrt(picked.pow(2).mean(-1, keepdim=True) + eps) * weight).to(out.dtype))
+
+
 def add_tanhnorm(h, branches, weight, bias, alpha, out, rows=None, branch_norm=None):
     total = h.clone()
     summed = torch.zeros_like(h)
@@ -536,8 +561,9 @@ def moe_route(logits, num_experts, top_k, correction, scale, eps, shared_gate, r
         picked, chosen = torch.topk(biased, top_k, dim=-1)
         gate = torch.sigmoid(_f(logits[:, num_experts])) if shared_gate else None
         return chosen.to(torch.int32), torch.softmax(picked, dim=-1) * scale, gate
-    scores = torch.softmax(_f(logits[:, :num_experts]), dim=-1)
-    choice = scores + correction
+    logits_only = _f(logits[:, :num_experts])
+    scores = torch.sigmoid(logits_only) if routing == "sigmoid_then_top" else torch.softmax(logits_only, dim=-1)
+    choice = scores if correction is None else scores + correction
     if groups:
         size = num_experts // groups
         best = choice.reshape(-1, groups, size).amax(dim=-1)
@@ -552,13 +578,14 @@ def moe_route(logits, num_experts, top_k, correction, scale, eps, shared_gate, r
 
 
 class MoePlan:
-    def __init__(self, chosen, num_experts, pad=16):
+    def __init__(self, chosen, num_experts, pad=16, weights=None):
         tokens, top_k = chosen.shape
         self.pad, self.tokens, self.top_k = pad, tokens, top_k
         self.capacity = -(-(tokens * top_k + num_experts * (pad - 1)) // pad) * pad
         self.source = torch.full((self.capacity,), -1, dtype=torch.int32)
         self.place = torch.full((tokens * top_k,), -1, dtype=torch.int32)
         self.tile_expert = torch.full((self.capacity // pad,), -1, dtype=torch.int32)
+        self.place_weight = None if weights is None else torch.zeros(self.capacity)
         cursor = 0
         flat = chosen.reshape(-1)
         for expert in range(num_experts):
@@ -566,16 +593,18 @@ class MoePlan:
             for index, entry in enumerate(entries.tolist()):
                 self.source[cursor + index] = entry // top_k
                 self.place[entry] = cursor + index
+                if weights is not None:
+                    self.place_weight[cursor + index] = weights.reshape(-1)[entry]
             tiles = -(-len(entries) // pad)
             self.tile_expert[cursor // pad:cursor // pad + tiles] = expert
             cursor += tiles * pad
 
 
-def moe_plan(chosen, num_experts, pad=None):
-    return MoePlan(chosen, num_experts, pad or 16)
+def moe_plan(chosen, num_experts, pad=None, weights=None):
+    return MoePlan(chosen, num_experts, pad or 16, weights)
 
 
-def moe_expert_gemm(x, plan, weight, out, gather, glu, squared_relu=False):
+def moe_expert_gemm(x, plan, weight, out, gather, glu, squared_relu=False, row_scale=None):
     out.zero_()
     for tile in range(plan.tile_expert.numel()):
         expert = int(plan.tile_expert[tile])
@@ -586,6 +615,8 @@ def moe_expert_gemm(x, plan, weight, out, gather, glu, squared_relu=False):
             if source < 0:
                 continue
             row = _f(x[source if gather else place])
+            if row_scale is not None:
+                row = row * row_scale[place]
             sums = _f(weight[expert]) @ row
             if glu is not None:
                 inner = sums.numel() // 2
@@ -609,9 +640,9 @@ ROUTE_PLAN_TOKENS = 64
 
 
 def moe_route_plan(logits, num_experts, top_k, correction, scale, eps, shared_gate, *, experts_with_matrices, pad=None,
-                   **how):
+                   place_weights=False, **how):
     chosen, weights, gate = moe_route(logits, num_experts, top_k, correction, scale, eps, shared_gate, **how)
-    return chosen, weights, gate, MoePlan(chosen, experts_with_matrices, pad or 16)
+    return chosen, weights, gate, MoePlan(chosen, experts_with_matrices, pad or 16, weights if place_weights else None)
 
 
 def into_the_stream(rows, tail):
@@ -627,7 +658,7 @@ def moe_combine(down, plan, weights, shared_rows, shared_gate, out, own_rows=Non
     rows = down[places.clamp(min=0)]
     own = torch.zeros((plan.tokens, down.shape[1])) if own_rows is None else _f(own_rows)
     rows = torch.where((places < 0)[:, :, None], own[:, None, :], rows)
-    total = (rows * weights[:, :, None]).sum(dim=1)
+    total = rows.sum(dim=1) if weights is None else (rows * weights[:, :, None]).sum(dim=1)
     if shared_rows is not None:
         total = total + (1.0 if shared_gate is None else shared_gate[:, None]) * _f(shared_rows)
     if tail is not None:
@@ -646,7 +677,7 @@ NAMES = ["fused_gemm_split", "add_partials_rmsnorm", "prefill_attention_supporte
          "add_scaled_rmsnorm", "polynorm", "tanh_rows", "head_norm_gate", "linear_state_scan", "linear_chunk_supported",
          "embed_bigram", "stream_add", "add_layernorm", "add_tanhnorm", "clamped_glu", "latent_prepare", "head_linear", "rotate_heads",
          "latent_attention_supported", "moe_route", "moe_route_plan", "moe_plan", "moe_expert_gemm", "moe_combine", "cast_rows",
-         "attention_prepare", "normed_sum"]
+         "attention_prepare", "normed_sum", "add_normed_rmsnorm"]
 
 
 def install(monkeypatch):
