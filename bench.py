@@ -4,8 +4,8 @@ MI355X.
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--dtype bf16|f32] [--layers L]
     python bench.py --workload serving [--shape 0.5b|7b|34b]
     python bench.py --microbench
-    python bench.py --design mukutar|lutosun|motolix|pemarax|pipizen [--shape 0.5b|7b] 
-        [--beside falcon_h1|lutosun|mukutar] [--layers L] [--window W] [--only DESIGN|falcon_h1]
+    python bench.py --design mukutar|lutosun|motolix|pemarax|pipizen|sazavik [--shape 0.5b|7b]
+        [--beside falcon_h1|DESIGN] [--layers L] [--window W] [--only DESIGN|falcon_h1]
 
 One JSON line: ``value`` = decoded tokens a second at batch 8 with every request at a
 2,048-token context (a step = one decode step of the whole batch: model, greedy sampling,
@@ -40,8 +40,11 @@ convolutions behind its projections, kept first tokens and a sink; two of window
 attention beside a Mamba-2 mixer, their outputs normed each; experts without a gate on every layer), and ``--design
 pipizen`` for a Pipizen-shaped one (layers in turn: latent attention with sinks, lightning attention, latent attention
 that reads the rows of the layer two before it, lightning attention; a tanh norm before and behind every branch;
-grouped routing with identity experts and a shared one on three layers of four, the fourth dense), with ``--beside
-lutosun`` or ``--beside mukutar`` beside the Lutosun- or Mukutar-shaped model of equal sizes instead of the Falcon-H1
+grouped routing with identity experts and a shared one on three layers of four, the fourth dense), and ``--design
+sazavik`` for a Sazavik-shaped one (layers in turn: chunked attention with sinks and a gate on its outputs, chunked
+attention in larger chunks, windowed attention with a linear distance bias and a gate, the same on the keys of the layer
+before it; an RMS norm before and behind every branch; clamped dense feed-forwards and sigmoid-routed experts beside a
+shared one in turn), with ``--beside`` another of the designs in its shape of equal sizes instead of the Falcon-H1
 shape.  The default workload and its line are not touched by any of them.
 
 ``--workload serving`` runs whole requests through the scheduler and the sampler instead
@@ -266,11 +269,44 @@ def pipizen_shape(shape: dict, layers: int) -> dict:
     return {"architecture": "Pipizen", "width": width, "vocab": shape["vocab_size"], "norm": {"eps": 1e-5}, "layers": listed}
 
 
+def sazavik_shape(shape: dict, layers: int, window: int) -> dict:
+    """A Sazavik configuration with the sizes of a Falcon-H1 ``shape``: the same width, vocabulary, heads and head size.
+    Layers in turn: attention with sinks and an output gate in chunks of one and a half windows (half a head turned),
+    attention in chunks of four windows (the whole head turned), windowed attention with a linear distance bias and an
+    output gate, and the same on the keys and values of the layer before it; in turn the dense feed-forward and sixteen
+    experts a quarter as wide, of which a token uses three beside a shared one of their width (as many products a token)."""
+    width, dim = shape["hidden_size"], shape["head_dim"]
+    sizes = {"heads": shape["num_attention_heads"], "kv_heads": shape["num_key_value_heads"], "dim": dim, "vdim": dim,
+             "scale": dim ** -0.5}
+    chunked = {"type": "attention", "mixer": dict(sizes, mask={"size": window + window // 2}, rot={"base": 1e5, "dims": dim // 2})}
+    wide = {"type": "attention_2", "mixer": dict(sizes, mask={"size": 4 * window}, rot={"base": 1e6, "dims": dim})}
+    distant = dict(sizes, mask={"size": window}, q_temp={"coef": 0.1, "every": 1024})
+    expert = shape["intermediate_size"] // 4
+    dense = {"kind": "dense", "ff": shape["intermediate_size"], "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": expert}, "router": {"experts": 16, "top": 3}, "shared": {"ff": expert}}
+    listed = []
+    for index in range(layers):
+        turn = index % 4
+        if turn < 2:
+            layer = chunked if turn == 0 else wide
+        else:
+            layer = {"type": "attention_3", "mixer": distant if turn == 2 else dict(distant, kv_from=index - 1)}
+        listed.append(dict(layer, mlp=moe if turn % 2 else dense))
+    return {"architecture": "Sazavik", "width": width, "vocab": shape["vocab_size"], "norm": {"eps": 1e-5},
+            "logit_softcap": 30.0, "layers": listed}
+
+
+# the designs beside Falcon-H1: configuration from (shape, layers, window)
+DESIGNS = {"mukutar": mukutar_shape, "lutosun": lambda shape, layers, window: lutosun_shape(shape, layers),
+           "motolix": lambda shape, layers, window: motolix_shape(shape, layers), "pemarax": pemarax_shape,
+           "pipizen": lambda shape, layers, window: pipizen_shape(shape, layers), "sazavik": sazavik_shape}
+
+
 def design_points(args) -> int:
     """Prompt and decode steps of a model of another design with the sizes of a Falcon-H1 shape, and of that shape."""
     import torch
     from macllm_infer_amd import Engine, Lane
-    from macllm_infer_amd.config import FalconH1Config, LutosunConfig, MotolixConfig, MukutarConfig, PemaraxConfig, PipizenConfig
+    from macllm_infer_amd.config import FalconH1Config, config_from_dict
     from macllm_infer_amd.sampling import GREEDY, Sampler, SamplerRow
     from macllm_infer_amd.weights.random_init import random_tensors
 
@@ -278,22 +314,10 @@ def design_points(args) -> int:
     layers = args.layers or 12
     storage = torch.bfloat16 if args.dtype == "bf16" else torch.float32
     element = 2 if args.dtype == "bf16" else 4
-    if args.design == "lutosun":
-        configs = {"lutosun": LutosunConfig.from_dict(lutosun_shape(shape, layers))}
-    elif args.design == "motolix":
-        configs = {"motolix": MotolixConfig.from_dict(motolix_shape(shape, layers))}
-    elif args.design == "pemarax":
-        configs = {"pemarax": PemaraxConfig.from_dict(pemarax_shape(shape, layers, args.window))}
-    elif args.design == "pipizen":
-        configs = {"pipizen": PipizenConfig.from_dict(pipizen_shape(shape, layers))}
-    else:
-        configs = {"mukutar": MukutarConfig.from_dict(mukutar_shape(shape, layers, args.window))}
-    # beside it the Falcon-H1 shape, or another design that shares its mechanisms (latent attention and routed
-    # experts: lutosun; a matrix-valued state with a fixed decay: mukutar)
-    if args.beside == "lutosun" and args.design != "lutosun":
-        configs["lutosun"] = LutosunConfig.from_dict(lutosun_shape(shape, layers))
-    elif args.beside == "mukutar" and args.design != "mukutar":
-        configs["mukutar"] = MukutarConfig.from_dict(mukutar_shape(shape, layers, args.window))
+    configs = {args.design: config_from_dict(DESIGNS[args.design](shape, layers, args.window))}
+    # beside it the Falcon-H1 shape, or another design that shares its mechanisms
+    if args.beside != "falcon_h1" and args.beside != args.design:
+        configs[args.beside] = config_from_dict(DESIGNS[args.beside](shape, layers, args.window))
     else:
         configs["falcon_h1"] = FalconH1Config.from_dict(dict(shape, num_hidden_layers=layers))
     batches = [] if args.prefill_only else ([args.batch] if args.skip_points else sorted({1, args.batch, 64}))
@@ -447,15 +471,15 @@ def main() -> int:
                         help="steps: the headline decode and prefill steps; serving: whole requests through the scheduler")
     parser.add_argument("--microbench", action="store_true",
                         help="only this GPU's streaming read and read-modify-write bandwidth")
-    parser.add_argument("--design", default=None, choices=["mukutar", "lutosun", "motolix", "pemarax", "pipizen"],
+    parser.add_argument("--design", default=None, choices=sorted(DESIGNS),
                         help="measure a model of this design with the sizes of --shape (12 layers unless --layers) beside "
                              "the Falcon-H1 shape of equal sizes, instead of the headline workload")
     parser.add_argument("--window", type=int, default=1024, help="--design: the attention layers' window")
-    parser.add_argument("--only", default=None, choices=["mukutar", "lutosun", "motolix", "pemarax", "pipizen", "falcon_h1"],
+    parser.add_argument("--only", default=None, choices=sorted(DESIGNS) + ["falcon_h1"],
                         help="--design: one of the two models")
-    parser.add_argument("--beside", default="falcon_h1", choices=["falcon_h1", "lutosun", "mukutar"],
-                        help="--design: the model measured beside it (the Falcon-H1 shape, or the Lutosun- or "
-                             "Mukutar-shaped model of equal sizes, where one of these shares more of its mechanisms)")
+    parser.add_argument("--beside", default="falcon_h1", choices=["falcon_h1"] + sorted(DESIGNS),
+                        help="--design: the model measured beside it (the Falcon-H1 shape, or a model of another design "
+                             "of equal sizes, where one of these shares more of its mechanisms)")
     parser.add_argument("--write-config", default=None, metavar="PATH",
                         help="write the config.json of --shape / --layers there and exit (what "
                              "utils.kernel_trace --config reads)")
@@ -468,16 +492,8 @@ def main() -> int:
     if args.write_config:
         shape = SHAPES[args.shape]
         with open(args.write_config, "w") as handle:
-            if args.design == "mukutar" and args.only != "falcon_h1":
-                json.dump(mukutar_shape(shape, args.layers or 12, args.window), handle)
-            elif args.design == "lutosun" and args.only != "falcon_h1":
-                json.dump(lutosun_shape(shape, args.layers or 12), handle)
-            elif args.design == "motolix" and args.only != "falcon_h1":
-                json.dump(motolix_shape(shape, args.layers or 12), handle)
-            elif args.design == "pemarax" and args.only != "falcon_h1":
-                json.dump(pemarax_shape(shape, args.layers or 12, args.window), handle)
-            elif args.design == "pipizen" and args.only != "falcon_h1":
-                json.dump(pipizen_shape(shape, args.layers or 12), handle)
+            if args.design and args.only != "falcon_h1":
+                json.dump(DESIGNS[args.only or args.design](shape, args.layers or 12, args.window), handle)
             else:
                 layers = args.layers or (12 if args.design else shape["num_hidden_layers"])
                 json.dump(dict(shape, num_hidden_layers=layers), handle)

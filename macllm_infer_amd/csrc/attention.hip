@@ -1364,10 +1364,10 @@ extern "C" int mi_prefill_attention_forms(const void* q, long q_ld, int Hq, int 
       nullptr, dv, head_scales, score_bias
 #define SIGMOID_CASE(DH_, NSET_)                                                                               \
   if (sigmoid && dh == DH_ && nset == NSET_)                                                                   \
-    prefill_attention_kernel<DH_, NSET_, false, DH_, true, false><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(FORM_ARGS);
+    prefill_attention_kernel<DH_, NSET_, BIAS_NONE, DH_, true, false><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(FORM_ARGS);
 #define PADDED_CASE(DH_, DV_, NSET_)                                                                           \
   if (!sigmoid && dh == DH_ && width == DV_ && nset == NSET_)                                                  \
-    prefill_attention_kernel<DH_, NSET_, false, DV_, false, true><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(FORM_ARGS);
+    prefill_attention_kernel<DH_, NSET_, BIAS_NONE, DV_, false, true><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(FORM_ARGS);
   SIGMOID_CASE(64, 1) SIGMOID_CASE(64, 2) SIGMOID_CASE(64, 3) SIGMOID_CASE(64, 4)
   SIGMOID_CASE(128, 1) SIGMOID_CASE(128, 2)
   PADDED_CASE(64, 32, 1) PADDED_CASE(64, 32, 2) PADDED_CASE(64, 32, 3) PADDED_CASE(64, 32, 4)
@@ -1413,22 +1413,20 @@ extern "C" int mi_prefill_attention(const void* q, long q_ld, int Hq, int Hkv, i
   const int nset = (G + passes - 1) / passes;
   if (n_tiles > (1 << 28)) return ERR_UNSUPPORTED_SIZE;
   const dim3 grid(4 * n_tiles, Hkv, passes);
-  const bool extras = log_bias != nullptr || sinks != nullptr || slopes != nullptr;
+#define PREFILL_LAUNCH(DH_, NSET_, BIAS_)                                                                      \
+  prefill_attention_kernel<DH_, NSET_, BIAS_><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(                     \
+      (const bf16_t*)q, q_ld, Hq, Hkv, (const bf16_t*)k_base, (const bf16_t*)v_base, page_stride, page_size,  \
+      block_tables, max_pages, tiles, cu_seqlens, start_pos, scale, window, (bf16_t*)out, out_ld, log_bias, sinks, \
+      DH_, nullptr, nullptr, kept, slopes, (const bf16_t*)gate, gate_ld)
 #define PREFILL_CASE(DH_, NSET_)                                                                              \
   if (dh == DH_ && nset == NSET_) {                                                                           \
-    if (extras)                                                                                               \
-      prefill_attention_kernel<DH_, NSET_, true><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(                  \
-          (const bf16_t*)q, q_ld, Hq, Hkv, (const bf16_t*)k_base, (const bf16_t*)v_base, page_stride, page_size, \
-          block_tables, max_pages, tiles, cu_seqlens, start_pos, scale, window, (bf16_t*)out, out_ld, log_bias, sinks, \
-          DH_, nullptr, nullptr, kept, slopes, (const bf16_t*)gate, gate_ld);                                 \
-    else                                                                                                      \
-      prefill_attention_kernel<DH_, NSET_><<<grid, PREFILL_WAVES * WAVE, 0, stream>>>(                        \
-          (const bf16_t*)q, q_ld, Hq, Hkv, (const bf16_t*)k_base, (const bf16_t*)v_base, page_stride, page_size, \
-          block_tables, max_pages, tiles, cu_seqlens, start_pos, scale, window, (bf16_t*)out, out_ld, nullptr, \
-          nullptr, DH_, nullptr, nullptr, kept, nullptr, (const bf16_t*)gate, gate_ld);                       \
+    if (log_bias) PREFILL_LAUNCH(DH_, NSET_, BIAS_LOG);                                                       \
+    else if (slopes) PREFILL_LAUNCH(DH_, NSET_, BIAS_LINEAR);                                                 \
+    else PREFILL_LAUNCH(DH_, NSET_, BIAS_NONE);                                                               \
   }
   PREFILL_CASE(64, 1) PREFILL_CASE(64, 2) PREFILL_CASE(64, 3) PREFILL_CASE(64, 4)
-  PREFILL_CASE(128, 1) PREFILL_CASE(128, 2) PREFILL_CASE(128, 3) PREFILL_CASE(128, 4)
+  PREFILL_CASE(128, 1) PREFILL_CASE(128, 2)
+#undef PREFILL_LAUNCH
 #undef PREFILL_CASE
   RETURN_IF_LAUNCH_FAILED();
   return 0;

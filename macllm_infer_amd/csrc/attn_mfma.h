@@ -116,14 +116,13 @@ __device__ __forceinline__ void attn_load(AttnFragments<DH, STEPS, DV>& f, int k
   }
 }
 
-// A bias on the scores that grows with the logarithm of the distance: score -= r1 * ln(1 + r2 * (position - key)),
-// one (r1, r2) for each set of columns (a query head).  In units of log2, where the scores live, that is
-// r1 * log2(1 + r2 * distance).  ``linear``: a bias that grows with the distance itself, score -= slope * distance
-// (``slope`` in units of log2).  Neither: no bias (the kernels that know none pass the default).
+// A bias on the scores by the distance between query and key, one for each set of columns (a query head).  BIAS_LOG:
+// score -= r1 * ln(1 + r2 * distance), in units of log2, where the scores live, r1 * log2(1 + r2 * distance); BIAS_LINEAR:
+// score -= slope * distance (``slope`` in units of log2).  Which one it is belongs to the kernel's type: the loops over
+// the keys have no branch for it.
+enum { BIAS_NONE = 0, BIAS_LOG = 1, BIAS_LINEAR = 2 };
 template <int NSET>
-struct AttnLogBias {
-  bool on = false;
-  bool linear = false;
+struct AttnBias {
   float r1[NSET];
   float r2[NSET];
   float slope[NSET];
@@ -142,11 +141,11 @@ struct AttnGate {
 // and lies inside the run (steps away from the diagonal, the window's edge and the run's end):
 // no masks are computed.
 // SIGMOID: the weights of ``gate`` instead of the softmax (acc.m and acc.l stay as they were cleared).
-template <int DH, int NSET, int STEPS, bool MASKED = true, bool BIASED = false, int DV = DH, bool SIGMOID = false>
+template <int DH, int NSET, int STEPS, bool MASKED = true, int BIAS = BIAS_NONE, int DV = DH, bool SIGMOID = false>
 __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc, AttnFragments<DH, STEPS, DV>& f,
                                              const mfma_bf16x8 (&q_frag)[NSET][DH / 32],
                                              const int (&col_pos)[NSET], const int (&col_first)[NSET], float scale, int k00,
-                                             int key_hi, const AttnLogBias<NSET>& bias = AttnLogBias<NSET>(),
+                                             int key_hi, const AttnBias<NSET>& bias = AttnBias<NSET>(),
                                              const AttnGate<NSET>* gate = nullptr, int kept = 0) {
   const int lane = threadIdx.x & (WAVE - 1);
   const int q = lane / 16;
@@ -184,29 +183,23 @@ __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc,
           score[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.k[st][t][kk], q_frag[s][kk], score[t], 0, 0, 0);
       }
       // scores in units of log2: s * scale * log2(e), so that the exponentials are bare v_exp
-      if (BIASED) {
-        // the biased scores, already in units of log2 (the scale below is then one); a key past the column's
-        // position gives a logarithm of anything, which the mask replaces
-        if (bias.on) {                 // the same for every lane
+      // the biased scores are already in units of log2 (the scale below is then one); a key past the column's position
+      // gets a bias of anything, which the mask replaces
+      if (BIAS == BIAS_LOG) {
 #pragma unroll
-          for (int t = 0; t < 2; ++t)
+        for (int t = 0; t < 2; ++t)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              const float distance = (float)(col_pos[s] - (k0 + 16 * t + 4 * q + i));
-              score[t][i] = fmaf(score[t][i], scale_log2, -bias.r1[s] * __log2f(fmaf(bias.r2[s], fmaxf(distance, 0.f), 1.f)));
-            }
-        } else if (bias.linear) {
+          for (int i = 0; i < 4; ++i) {
+            const float distance = (float)(col_pos[s] - (k0 + 16 * t + 4 * q + i));
+            score[t][i] = fmaf(score[t][i], scale_log2, -bias.r1[s] * __log2f(fmaf(bias.r2[s], fmaxf(distance, 0.f), 1.f)));
+          }
+      }
+      if (BIAS == BIAS_LINEAR) {
+        const float first = -bias.slope[s] * (float)(col_pos[s] - (k0 + 4 * q));     // of the lane's first key
 #pragma unroll
-          for (int t = 0; t < 2; ++t)
+        for (int t = 0; t < 2; ++t)
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
-              score[t][i] = fmaf(score[t][i], scale_log2, -bias.slope[s] * (float)(col_pos[s] - (k0 + 16 * t + 4 * q + i)));
-        } else {                       // a caller of this form for its sink alone: the scale, no logarithms
-#pragma unroll
-          for (int t = 0; t < 2; ++t)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) score[t][i] *= scale_log2;
-        }
+          for (int i = 0; i < 4; ++i) score[t][i] = fmaf(score[t][i], scale_log2, fmaf(bias.slope[s], (float)(16 * t + i), first));
       }
       if (MASKED) {
         // visible keys of the column: first_visible .. min(position, last_key); relative to the step
@@ -251,7 +244,7 @@ __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc,
                              fmaxf(fmaxf(score[1][0], score[1][1]), fmaxf(score[1][2], score[1][3])));
       step_max = fmaxf(step_max, __shfl_xor(step_max, 16, WAVE));
       step_max = fmaxf(step_max, __shfl_xor(step_max, 32, WAVE));
-      if (!BIASED) step_max *= scale_log2;                           // scale > 0: the maximum stays the maximum
+      if (BIAS == BIAS_NONE) step_max *= scale_log2;                           // scale > 0: the maximum stays the maximum
       const float m_new = fmaxf(acc.m[s], step_max);
       const float m_safe = m_new == -INFINITY ? 0.f : m_new;       // nothing visible yet
       const float correction = __builtin_amdgcn_exp2f(acc.m[s] - m_safe);
@@ -262,7 +255,7 @@ __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc,
       for (int t = 0; t < 2; ++t)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float p = __builtin_amdgcn_exp2f(BIASED ? score[t][i] - m_safe : fmaf(score[t][i], scale_log2, -m_safe));
+          const float p = __builtin_amdgcn_exp2f(BIAS != BIAS_NONE ? score[t][i] - m_safe : fmaf(score[t][i], scale_log2, -m_safe));
           sum += p;
           p_frag[4 * t + i] = (bf16_t)p;
         }
@@ -288,13 +281,13 @@ __device__ __forceinline__ void attn_compute(AttnAccumulator<DH, NSET, DV>& acc,
 // of them hold queries and the caller knows (the same value in every lane), else -1.
 // SIGMOID (with ``gate``), PADDED (with cache.value_dim) and PADDED_KEYS (with cache.key_dim): see attn_compute and
 // attn_load; not PIPELINED.
-template <int DH, int NSET, int STEPS, bool PIPELINED = false, bool BIASED = false, int DV = DH, bool SIGMOID = false,
+template <int DH, int NSET, int STEPS, bool PIPELINED = false, int BIAS = BIAS_NONE, int DV = DH, bool SIGMOID = false,
           bool PADDED = false, bool PADDED_KEYS = false>
 __device__ __forceinline__ void attend_keys(AttnAccumulator<DH, NSET, DV>& acc,
                                             const mfma_bf16x8 (&q_frag)[NSET][DH / 32],
                                             const int (&col_pos)[NSET], int window, float scale, int key_lo,
                                             int key_hi, const AttnCache& cache, int min_pos = -1, int max_pos = -1,
-                                            const AttnLogBias<NSET>& bias = AttnLogBias<NSET>(),
+                                            const AttnBias<NSET>& bias = AttnBias<NSET>(),
                                             const AttnGate<NSET>* gate = nullptr, int kept = 0) {
   const int last_key = key_hi - 1;
   constexpr int ROUND = 32 * STEPS;
@@ -308,10 +301,10 @@ __device__ __forceinline__ void attend_keys(AttnAccumulator<DH, NSET, DV>& acc,
     attn_load<DH, STEPS, DV>(even, key_lo, last_key, cache);
     for (int k00 = key_lo; k00 < key_hi; k00 += 2 * ROUND) {
       attn_load<DH, STEPS, DV>(odd, k00 + ROUND, last_key, cache);
-      attn_compute<DH, NSET, STEPS, true, false, DV>(acc, even, q_frag, col_pos, col_first, scale, k00, key_hi);
+      attn_compute<DH, NSET, STEPS, true, BIAS_NONE, DV>(acc, even, q_frag, col_pos, col_first, scale, k00, key_hi);
       attn_load<DH, STEPS, DV>(even, k00 + 2 * ROUND, last_key, cache);
       if (k00 + ROUND < key_hi)
-        attn_compute<DH, NSET, STEPS, true, false, DV>(acc, odd, q_frag, col_pos, col_first, scale, k00 + ROUND, key_hi);
+        attn_compute<DH, NSET, STEPS, true, BIAS_NONE, DV>(acc, odd, q_frag, col_pos, col_first, scale, k00 + ROUND, key_hi);
     }
   } else {
     // rounds all of whose keys every column of the wave sees run without masks, in a loop of
@@ -322,13 +315,13 @@ __device__ __forceinline__ void attend_keys(AttnAccumulator<DH, NSET, DV>& acc,
     for (int k00 = key_lo; k00 < open_hi; k00 += ROUND) {
       AttnFragments<DH, STEPS, DV> f;
       attn_load<DH, STEPS, DV, PADDED, PADDED_KEYS>(f, k00, last_key, cache);
-      attn_compute<DH, NSET, STEPS, false, BIASED, DV, SIGMOID>(acc, f, q_frag, col_pos, col_first, scale, k00, key_hi, bias,
+      attn_compute<DH, NSET, STEPS, false, BIAS, DV, SIGMOID>(acc, f, q_frag, col_pos, col_first, scale, k00, key_hi, bias,
                                                                 gate);
     }
     for (int k00 = open_hi; k00 < key_hi; k00 += ROUND) {
       AttnFragments<DH, STEPS, DV> f;
       attn_load<DH, STEPS, DV, PADDED, PADDED_KEYS>(f, k00, last_key, cache);
-      attn_compute<DH, NSET, STEPS, true, BIASED, DV, SIGMOID>(acc, f, q_frag, col_pos, col_first, scale, k00, key_hi, bias,
+      attn_compute<DH, NSET, STEPS, true, BIAS, DV, SIGMOID>(acc, f, q_frag, col_pos, col_first, scale, k00, key_hi, bias,
                                                                gate, kept);
     }
   }

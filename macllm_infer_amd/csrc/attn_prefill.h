@@ -14,15 +14,15 @@
 #define PREFILL_WAVES 8
 #define PREFILL_FILL_BLOCKS 512   // two workgroups for each of the 256 compute units
 
-// EXTRAS: the scores lose log_bias[head] = (r1, r2) -> r1 * ln(1 + r2 * distance), and the softmax's denominator
-// holds one more term exp(sinks[head]) (either pointer may be null).
+// BIAS: BIAS_LOG, the scores lose log_bias[head] = (r1, r2) -> r1 * ln(1 + r2 * distance); BIAS_LINEAR, they lose
+// slopes[head] * distance.  sinks (may be null): one more term exp(sinks[head]) of the softmax's denominator.
 // DV: the width the values are computed with, the keys' or, PADDED, the next width of the launch's table above
 // value_dim, the width of the cached values and of a head's output (a multiple of 4).
 // SIGMOID: a visible key weighs sigmoid(score * scale * head_scales[head] + score_bias[head]) on its own (either
 // pointer may be null: 1 and 0); no maximum, no normalizer, the waves' partial sums are added as they are.
-// slopes (EXTRAS, in place of log_bias): score -= slopes[head] * distance.  PADDED_KEYS: the cached keys and the queries are
+// PADDED_KEYS: the cached keys and the queries are
 // key_dim wide, a multiple of 8 and at most DH.  out_gate: see output_gate (softmax weights; rows in pieces of four).
-template <int DH, int NSET, bool EXTRAS = false, int DV = DH, bool SIGMOID = false, bool PADDED = false,
+template <int DH, int NSET, int BIAS = BIAS_NONE, int DV = DH, bool SIGMOID = false, bool PADDED = false,
           bool PADDED_KEYS = false>
 __global__ void __launch_bounds__(PREFILL_WAVES * WAVE)
 prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hkv, const bf16_t* __restrict__ k_base,
@@ -92,17 +92,13 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hk
       gate.bias[s] = score_bias ? score_bias[head] : 0.f;
     }
   }
-  AttnLogBias<NSET> bias;
-  if (EXTRAS) {
-    bias.on = log_bias != nullptr;
-    bias.linear = slopes != nullptr;
+  AttnBias<NSET> bias;
 #pragma unroll
-    for (int s = 0; s < NSET; ++s) {
-      const int head = min(head0 + s, Hq - 1);
-      bias.slope[s] = slopes ? slopes[head] * 1.4426950408889634f : 0.f;
-      bias.r1[s] = log_bias ? log_bias[2 * head] : 0.f;
-      bias.r2[s] = log_bias ? log_bias[2 * head + 1] : 0.f;
-    }
+  for (int s = 0; s < NSET; ++s) {
+    const int head = min(head0 + s, Hq - 1);
+    bias.slope[s] = BIAS == BIAS_LINEAR ? slopes[head] * 1.4426950408889634f : 0.f;
+    bias.r1[s] = BIAS == BIAS_LOG ? log_bias[2 * head] : 0.f;
+    bias.r2[s] = BIAS == BIAS_LOG ? log_bias[2 * head + 1] : 0.f;
   }
   AttnCache cache;
   cache.k_base = k_base;
@@ -128,7 +124,7 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hk
       wave_pages[wave][lane] = cache_pages[min(first_page + lane, max_pages - 1)];
       cache.pages = wave_pages[wave];
       cache.base_page = first_page;
-      attend_keys<DH, NSET, PREFILL_STEPS, false, EXTRAS, DV, SIGMOID, PADDED, PADDED_KEYS>(
+      attend_keys<DH, NSET, PREFILL_STEPS, false, BIAS, DV, SIGMOID, PADDED, PADDED_KEYS>(
           acc, q_frag, col_pos, window, scale, part_lo, part_hi, cache, full_tile ? first_position : -1, last_position,
           bias, &gate, kept);
       part_lo = part_hi;
@@ -141,6 +137,15 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hk
   // merge: set s is finished by wave s
 #pragma unroll
   for (int s = 0; s < NSET; ++s) {
+    // the gate of the outputs this wave will write, asked for ahead of the exchange through LDS
+    mfma_bf16x4 gate_piece[DV / 16];
+    const bool gated = !SIGMOID && out_gate && wave == s % PREFILL_WAVES && col_pos[s] >= 0;
+    if (gated) {
+      const bf16_t* gate_row = out_gate + (long)token * gate_ld + (long)(head0 + s) * value_dim;
+#pragma unroll
+      for (int dt = 0; dt < DV / 16; ++dt)
+        if (!PADDED || 16 * dt + 4 * qd < value_dim) gate_piece[dt] = *reinterpret_cast<const mfma_bf16x4*>(gate_row + 16 * dt + 4 * qd);
+    }
     __syncthreads();
     part[wave][0][lane] = acc.m[s];
     part[wave][1][lane] = acc.l[s];
@@ -171,7 +176,7 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hk
 #pragma unroll
     for (int w = 0; w < PREFILL_WAVES; ++w) m = fmaxf(m, part[w][0][lane]);
     // the sink, in the scores' units of log2: it may be the largest term
-    const float sink = (EXTRAS && sinks) ? sinks[min(head0 + s, Hq - 1)] * 1.4426950408889634f : -INFINITY;
+    const float sink = sinks ? sinks[min(head0 + s, Hq - 1)] * 1.4426950408889634f : -INFINITY;
     m = fmaxf(m, sink);
     float factor[PREFILL_WAVES];
     float l = 0.f;
@@ -183,11 +188,10 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hk
     }
     l += __shfl_xor(l, 16, WAVE);
     l += __shfl_xor(l, 32, WAVE);
-    if (EXTRAS && sinks) l += __builtin_amdgcn_exp2f(sink - m);       // once for the column: no key, no value
+    if (sinks) l += __builtin_amdgcn_exp2f(sink - m);       // once for the column: no key, no value
     if (col_pos[s] < 0) continue;
     const float inverse = 1.f / l;
     bf16_t* o = out + (long)token * out_ld + (long)(head0 + s) * value_dim;
-    const bf16_t* gate_row = out_gate ? out_gate + (long)token * gate_ld + (long)(head0 + s) * value_dim : nullptr;
 #pragma unroll
     for (int dt = 0; dt < DV / 16; ++dt) {
       if (PADDED && 16 * dt + 4 * qd >= value_dim) continue;
@@ -199,10 +203,9 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, int Hk
         for (int w = 0; w < PREFILL_WAVES; ++w) value[i] += part[w][2 + 4 * dt + i][lane] * factor[w];
         value[i] *= inverse;
       }
-      if (gate_row) {
-        const mfma_bf16x4 piece = *reinterpret_cast<const mfma_bf16x4*>(gate_row + 16 * dt + 4 * qd);
+      if (gated) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) value[i] *= 1.0f / (1.0f + __expf(-(float)piece[i]));
+        for (int i = 0; i < 4; ++i) value[i] *= __frcp_rn(1.0f + __expf(-(float)gate_piece[dt][i]));
       }
       mfma_bf16x4 packed;
 #pragma unroll

@@ -137,7 +137,7 @@ _SIGNATURES = {
     "attention_widths": {
         "mi_prefill_attention_padded": [_c_ptr, _c_long, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_long, _c_int,
                                         _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int, _c_int, _c_ptr,
-                                        _c_long, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_long, _c_ptr],
+                                        _c_long, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_long, _c_ptr],
     },
     "mamba2": {
         "mi_conv1d_silu": [_c_ptr, _c_int, _c_long, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
@@ -1501,10 +1501,12 @@ def prefill_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
     gate_ld = _gate_rows(gate, out, "prefill_attention")
     _need(gate is None or (gate_ld % 4 == 0 and gate.data_ptr() % 8 == 0), "prefill_attention: the gate's rows lie in pieces of four")
     own_width = head_dim in (64, 128) and value_dim == head_dim
+    _need(own_width or log_bias is None, "prefill_attention: the logarithmic bias comes with heads of 64 or 128 and values as wide")
     _check(_fn(*(("attention", "mi_prefill_attention") if own_width else ("attention_widths", "mi_prefill_attention_padded")))(
         _p(q), q_ld, num_heads, num_kv_heads, head_dim, *(() if own_width else (value_dim,)), _p(k_cache), _p(v_cache),
         page_stride, page_size, _p(block_tables), block_tables.shape[1], _p(query_tiles), query_tiles.shape[0],
-        _p(cu_seqlens), _p(start_pos), float(scale), span_code, int(max_seq_len or 0), _p(out), out_ld, _p(log_bias),
+        _p(cu_seqlens), _p(start_pos), float(scale), span_code, int(max_seq_len or 0), _p(out), out_ld,
+        *((_p(log_bias),) if own_width else ()),
         _p(sinks), int(keep_first), _p(slopes), _p(gate), gate_ld, _stream()), "prefill_attention")
 
 
