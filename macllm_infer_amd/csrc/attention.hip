@@ -250,6 +250,104 @@ attention_prepare_kernel(T* __restrict__ qkv, long ld, int Hq, int Hkv, int dh, 
   }
 }
 
+// The same where no norm spans a whole projection: everything is then head by head, and a wave makes one head ready by
+// itself (grid: tokens x fours of [q heads | k heads | v heads]), its elements in registers, a lane the elements lane,
+// lane + 64, ...; a pair's partner comes through the wave's own row of LDS.  The sums are the ones of the kernel above.
+#define PREPARE_WAVES 4
+#define PREPARE_PER_LANE 4       // heads of up to 256 dims
+#define PREPARE_HEADS_TOKENS 512
+template <typename T>
+__global__ void __launch_bounds__(PREPARE_WAVES * WAVE)
+attention_prepare_heads_kernel(T* __restrict__ qkv, long ld, int Hq, int Hkv, int dh, int dv, int values_from_keys,
+                               const int* __restrict__ positions, const float* __restrict__ inv_freq, int rotary_dim,
+                               int interleaved, float turn_scale, int head_norm, const float* __restrict__ q_head_weight,
+                               const float* __restrict__ k_head_weight, float head_eps, float temp_coef, int temp_every,
+                               const float* __restrict__ value_inv_freq, const int* __restrict__ slot_mapping,
+                               T* __restrict__ k_base, T* __restrict__ v_base, long page_stride, int page_size) {
+  __shared__ float rows[PREPARE_WAVES][WAVE * PREPARE_PER_LANE];
+  const long token = blockIdx.x;
+  const int lane = threadIdx.x & (WAVE - 1);
+  const int wave = threadIdx.x / WAVE;
+  const int index = blockIdx.y * PREPARE_WAVES + wave;              // q heads, k heads, v heads
+  if (index >= Hq + 2 * Hkv) return;                                 // (no barrier of the workgroup below)
+  const bool is_q = index < Hq;
+  const bool is_v = index >= Hq + Hkv;
+  const int kvh = is_v ? index - Hq - Hkv : index - Hq;
+  const int width = is_v ? dv : dh;
+  const int place = positions[token];
+  const float position = (float)place;
+  const int cell = slot_mapping ? slot_mapping[token] : -1;
+  T* row = qkv + token * ld;
+  T* from = row;
+  if (is_q) from += (long)index * dh;
+  else if (!is_v || values_from_keys) from += (long)(Hq + kvh) * dh;
+  else from += (long)(Hq + Hkv) * dh + (long)kvh * dv;
+  const float* weight = is_v ? nullptr : is_q ? q_head_weight : k_head_weight;
+  const int turned = is_v ? (value_inv_freq ? dv : 0) : (inv_freq ? rotary_dim : 0);
+  const float* frequencies = is_v ? value_inv_freq : inv_freq;
+  const float magnitude = is_v ? 1.0f : turn_scale;
+  const bool neighbours = !is_v && interleaved;
+  const int norm = is_v ? 0 : head_norm;
+  float x[PREPARE_PER_LANE], w[PREPARE_PER_LANE];
+#pragma unroll
+  for (int i = 0; i < PREPARE_PER_LANE; ++i) {
+    const int j = lane + WAVE * i;
+    x[i] = j < width ? to_float(from[j]) : 0.f;
+    w[i] = (weight && j < width) ? weight[j] : 1.f;
+  }
+  auto norm_head = [&]() {
+    float squares = 0.f;
+#pragma unroll
+    for (int i = 0; i < PREPARE_PER_LANE; ++i) squares = fmaf(x[i], x[i], squares);
+    const float rms = sqrtf(wave_sum(squares) / (float)dh + head_eps);
+#pragma unroll
+    for (int i = 0; i < PREPARE_PER_LANE; ++i) x[i] = weight ? x[i] / rms * w[i] : x[i] / rms;
+  };
+  if (norm == 1) norm_head();
+  if (turned > 0) {
+    const int half = turned / 2;
+    float* mine = rows[wave];
+#pragma unroll
+    for (int i = 0; i < PREPARE_PER_LANE; ++i) mine[lane + WAVE * i] = x[i];
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < PREPARE_PER_LANE; ++i) {
+      const int j = lane + WAVE * i;
+      if (j < turned) {
+        const int pair = neighbours ? j / 2 : (j < half ? j : j - half);
+        const bool first = neighbours ? (j & 1) == 0 : j < half;
+        const float partner = mine[neighbours ? (j ^ 1) : (first ? j + half : j - half)];
+        float sine, cosine;
+        sincosf(position * frequencies[pair], &sine, &cosine);
+        sine *= magnitude;
+        cosine *= magnitude;
+        x[i] = first ? x[i] * cosine - partner * sine : x[i] * cosine + partner * sine;
+      }
+    }
+  }
+  if (norm == 2) norm_head();
+  if (is_q) {
+    const float temperature = temp_every > 0 ? 1.0f + temp_coef * logf((float)((place + 1) / temp_every + 1)) : 1.0f;
+#pragma unroll
+    for (int i = 0; i < PREPARE_PER_LANE; ++i) {
+      const int j = lane + WAVE * i;
+      if (j < width) from[j] = from_float<T>(x[i] * temperature);
+    }
+    return;
+  }
+  if (cell < 0) return;
+  const int page = cell / page_size;
+  const int offset = cell - page * page_size;
+  T* to = is_v ? v_base + (long)page * page_stride + (long)kvh * dv * page_size + offset
+               : k_base + (long)page * page_stride + ((long)kvh * page_size + offset) * dh;
+  const int step = is_v ? page_size : 1;
+#pragma unroll
+  for (int i = 0; i < PREPARE_PER_LANE; ++i) {
+    const int j = lane + WAVE * i;
+    if (j < width) to[(long)j * step] = from_float<T>(x[i]);
+  }
+}
+
 extern "C" int mi_attention_prepare(void* qkv, int dtype, long ld, int T, int Hq, int Hkv, int dh, int dv,
                                     int values_from_keys, const int* positions, const float* inv_freq, int rotary_dim,
                                     int interleaved, float turn_scale,
@@ -268,6 +366,22 @@ extern "C" int mi_attention_prepare(void* qkv, int dtype, long ld, int T, int Hq
   if (ld < (long)(Hq + Hkv) * dh + (values_from_keys ? 0L : (long)Hkv * dv)) return ERR_BAD_ARGUMENT;
   if (slot_mapping && (!k_base || !v_base || page_size <= 0)) return ERR_BAD_ARGUMENT;
   if (!inv_freq) rotary_dim = 0;
+  // few tokens wait for a chain of loads, which is shortest head by head; many tokens share a row's turns
+  if (!q_norm && T <= PREPARE_HEADS_TOKENS && dh <= WAVE * PREPARE_PER_LANE && dv <= WAVE * PREPARE_PER_LANE) {
+    const int items = slot_mapping ? Hq + 2 * Hkv : Hq;      // without cells the keys and values go nowhere
+    const dim3 grid(T, (items + PREPARE_WAVES - 1) / PREPARE_WAVES);
+#define PREPARE_HEADS(T_)                                                                                                   \
+  attention_prepare_heads_kernel<T_><<<grid, PREPARE_WAVES * WAVE, 0, stream>>>(                                            \
+      (T_*)qkv, ld, Hq, slot_mapping ? Hkv : 0, dh, dv, values_from_keys, positions, inv_freq, rotary_dim, interleaved,     \
+      turn_scale, head_norm, q_head_weight, k_head_weight, head_eps, temp_coef, temp_every, value_inv_freq, slot_mapping,   \
+      (T_*)k_base, (T_*)v_base, page_stride, page_size)
+    if (dtype == DT_F32) PREPARE_HEADS(float);
+    else if (dtype == DT_BF16) PREPARE_HEADS(bf16_t);
+    else return ERR_BAD_ARGUMENT;
+#undef PREPARE_HEADS
+    RETURN_IF_LAUNCH_FAILED();
+    return 0;
+  }
   // the row, and (cosine, sine) of the keys' and the values' pairs
   const size_t lds = ((size_t)(Hq + Hkv) * dh + (size_t)Hkv * dv + (size_t)rotary_dim + (size_t)(dv / 2) * 2) * sizeof(float);
   if (lds > 64 * 1024) return ERR_UNSUPPORTED_SIZE;
@@ -906,6 +1020,7 @@ extern "C" int mi_paged_attention(const void* q, int dtype, long q_ld, int T, in
 #define DEC_THREADS 256
 #define DEC_WAVES (DEC_THREADS / WAVE)
 #define DEC_MAX_SPLIT 512
+#define DEC_AHEAD 4               // rounds of keys asked for at once
 #define DEC_MERGE_SPLITS 256     // splits whose factors the merge keeps in LDS
 
 struct alignas(16) bf16x8 {
@@ -984,36 +1099,42 @@ decode_attention_kernel(const bf16_t* __restrict__ q, long q_ld, int Hq, const b
     for (int j = 0; j < 8; ++j) qf[g][j] = (float)packed.v[j] * factor;
   }
 
-  // scores
-  for (int base = 0; base < count; base += KPB) {
-    const int local = base + wave * KPW + r;
-    const int key = range_lo + local;
-    const bool valid = local < count;
-    float s[G];
+  // scores, DEC_AHEAD rounds of keys at a time: their page ids, then their rows, are asked for together
+  for (int base0 = 0; base0 < count; base0 += DEC_AHEAD * KPB) {
+    int key[DEC_AHEAD], page[DEC_AHEAD];
+    bf16x8 packed[DEC_AHEAD];
 #pragma unroll
-    for (int g = 0; g < G; ++g) s[g] = 0.f;
-    if (valid && brings) {
-      const int page = table[key / page_size];
-      const int offset = key % page_size;
-      const bf16x8 packed = *reinterpret_cast<const bf16x8*>(
-          k_base + (long)page * page_stride + ((long)kvh * page_size + offset) * dh + c * 8);
-      float kf[8];
-#pragma unroll
-      for (int j = 0; j < 8; ++j) kf[j] = (float)packed.v[j];
-#pragma unroll
-      for (int g = 0; g < G; ++g)
-#pragma unroll
-        for (int j = 0; j < 8; ++j) s[g] = fmaf(qf[g][j], kf[j], s[g]);
+    for (int a = 0; a < DEC_AHEAD; ++a) {
+      key[a] = range_lo + min(base0 + a * KPB + wave * KPW + r, count - 1);      // (past the range: its last key again, dropped below)
+      page[a] = table[key[a] / page_size];
     }
 #pragma unroll
-    for (int offset = LPR / 2; offset > 0; offset >>= 1)
+    for (int a = 0; a < DEC_AHEAD; ++a)
+      packed[a] = *reinterpret_cast<const bf16x8*>(k_base + (long)page[a] * page_stride +
+                                                   ((long)kvh * page_size + key[a] % page_size) * dh + (brings ? c * 8 : 0));
 #pragma unroll
-      for (int g = 0; g < G; ++g) s[g] += __shfl_xor(s[g], offset, WAVE);
-    if (valid && c == 0) {
+    for (int a = 0; a < DEC_AHEAD; ++a) {
+      const int local = base0 + a * KPB + wave * KPW + r;
+      if (base0 + a * KPB >= count) break;                                       // the same for every lane
+      float s[G], kf[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) kf[j] = brings ? (float)packed[a].v[j] : 0.f;
 #pragma unroll
       for (int g = 0; g < G; ++g) {
-        const float score = fmaf(-slope_of[g], (float)(pos - key), s[g] + offset_of[g]);
-        s_lds[g][local] = (key >= first_key || key < kept) ? score : -INFINITY;
+        s[g] = 0.f;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) s[g] = fmaf(qf[g][j], kf[j], s[g]);
+      }
+#pragma unroll
+      for (int offset = LPR / 2; offset > 0; offset >>= 1)
+#pragma unroll
+        for (int g = 0; g < G; ++g) s[g] += __shfl_xor(s[g], offset, WAVE);
+      if (local < count && c == 0) {
+#pragma unroll
+        for (int g = 0; g < G; ++g) {
+          const float score = fmaf(-slope_of[g], (float)(pos - key[a]), s[g] + offset_of[g]);
+          s_lds[g][local] = (key[a] >= first_key || key[a] < kept) ? score : -INFINITY;
+        }
       }
     }
   }

@@ -104,10 +104,12 @@ def test_the_clamped_gate_in_the_product_s_epilogue(rows, width, inner):
     (5, 5, 7, 9, 0, False, "before_rotation", (-0.2, 1)), (6, 2, 128, 64, 32, True, "after_rotation", (0.1, 1000)),
     (2, 1, 250, 256, 250, False, None, (0.3, 7))])
 @pytest.mark.parametrize("alone", [False, True])
+@pytest.mark.parametrize("T", [21, 600])
 def test_a_row_is_made_ready_with_a_temperature_and_without_keys(dtype, Hq, Hkv, dh, dv, rotary, interleaved, head_norm,
-                                                                 temperature, alone):
-    """``alone``: a row of queries whose keys and values another layer has cached."""
-    T, page, pages = 21, 4, 9
+                                                                 temperature, alone, T):
+    """``alone``: a row of queries whose keys and values another layer has cached.  Few rows go head by head, many as
+    whole rows."""
+    page, pages = 4, T // 4 + 3
     kv = 0 if alone else Hkv
     width = (Hq + kv) * dh + kv * dv
     qkv = rand(T, width + 5, seed=1).to(dtype)
@@ -730,7 +732,7 @@ def drawn_configuration(seed):
     feed-forward, with and without a cap on the logits."""
     import random
     draw = random.Random(seed)
-    width = draw.choice([24, 40, 56, 64, 96, 128])
+    width = draw.choice([24, 36, 40, 50, 64, 96, 128])
     layers, own = [], []
     for index in range(draw.choice([3, 4, 5, 6])):
         reads = own and draw.random() < 0.35
