@@ -1198,14 +1198,17 @@ def linear_chunk_scan(u: torch.Tensor, *, q_col: int, k_col: int, v_col: int, nu
 SKINNY_ROWS = 16          # steps of up to this many rows take the skinny kernel in ``linear``
 
 
-def linear(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], keep_float32: bool = False) -> torch.Tensor:
+def linear(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], keep_float32: bool = False,
+           bias16: Optional[torch.Tensor] = None) -> torch.Tensor:
     """x [M, K] . weight[N, K]^T (+ bias float32 [N]) -> [M, N] in x's dtype, or, with
     ``keep_float32`` and no bias, in float32 whatever the operands are (the library writes its
     float32 sums without rounding them to bfloat16: the logits).
 
     float32 operands: the hand-written float32 FMA kernel (true 32-bit).  bfloat16 operands:
     the BLAS library with float32 accumulation.  A float32 weight with bfloat16 activations
-    (a tensor that was stored in 32-bit) runs in float32 and the result is rounded once."""
+    (a tensor that was stored in 32-bit) runs in float32 and the result is rounded once.
+    ``bias16``: the bias in bfloat16, if that holds the same numbers: the library's products of many rows then add it
+    to their float32 sums themselves."""
     _need(x.dim() == 2 and weight.dim() == 2 and x.shape[1] == weight.shape[1], "linear: shapes do not match")
     if weight.dtype == torch.float32:
         xf = x if x.dtype == torch.float32 else x.float()
@@ -1233,6 +1236,10 @@ def linear(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], 
         return torch.mm(x, weight.t(), out_dtype=torch.float32)
     if bias is None:
         return torch.mm(x, weight.t())
+    if bias16 is not None:
+        _need(bias16.dtype == torch.bfloat16 and bias16.numel() == weight.shape[0] and bias16.is_contiguous(),
+              "linear: bias16 must be bfloat16 [N]")
+        return torch.addmm(bias16, x, weight.t())
     # the bias stays float32: it is added to the product's float32 sums, and the result is rounded once
     _need(bias.dtype == torch.float32 and bias.numel() == weight.shape[0] and bias.is_contiguous(),
           "linear: bias must be float32 [N]")

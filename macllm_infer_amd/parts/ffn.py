@@ -51,6 +51,8 @@ class SwiGLU(FeedForward):
             self.gate_up.weight = self.gate_up.weight[order].contiguous()
             if self.gate_up.bias is not None:
                 self.gate_up.bias = self.gate_up.bias[order].contiguous()
+            if self.gate_up.bias16 is not None:
+                self.gate_up.bias16 = self.gate_up.bias16[order].contiguous()
 
     def gated_projections(self):
         if self.spec.activation != "silu":          # the fused decode kernels apply SiLU

@@ -42,7 +42,7 @@ class Linear:
         if scale is not None:
             weight = weight * scale.to(weight.device)
         self.weight = weight.to(keep).contiguous().to(build.device)
-        self.bias = None
+        self.bias = self.bias16 = None      # ``bias16``: the bias in bfloat16 where that changes none of its numbers
         if any(b is not None for b in biases):
             parts = [torch.zeros(w.shape[0], device=w.device) if b is None else b.to(torch.float32).reshape(-1)
                      for w, b in zip(weights, biases)]
@@ -51,10 +51,11 @@ class Linear:
             if scale is not None:
                 bias = bias * scale.reshape(-1).to(bias.device)
             self.bias = bias.contiguous().to(build.device)
+            if keep == torch.bfloat16 and bool((bias.to(torch.bfloat16).to(torch.float32) == bias).all()):
+                self.bias16 = self.bias.to(torch.bfloat16)
         self.out_features, self.in_features = self.weight.shape
 
     def __call__(self, x: torch.Tensor, rows: Optional[int] = None) -> torch.Tensor:
         """``rows``: use only the first ``rows`` output rows."""
-        if rows is None:
-            return ops.linear(x, self.weight, self.bias)
-        return ops.linear(x, self.weight[:rows], None if self.bias is None else self.bias[:rows])
+        part = lambda bias: bias if bias is None or rows is None else bias[:rows]
+        return ops.linear(x, self.weight if rows is None else self.weight[:rows], part(self.bias), bias16=part(self.bias16))

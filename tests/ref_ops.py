@@ -148,7 +148,7 @@ def add_partials_rmsnorm(h, partial, weight, eps, out):
         out.copy_((h / torch.sqrt(h.pow(2).mean(dim=-1, keepdim=True) + eps) * weight).to(out.dtype))
 
 
-def linear(x, weight, bias, keep_float32=False):
+def linear(x, weight, bias, keep_float32=False, bias16=None):
     y = _f(x) @ _f(weight).T
     if bias is not None:
         y = y + bias

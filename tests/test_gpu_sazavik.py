@@ -262,6 +262,20 @@ def test_weights_multiply_what_an_expert_is_given(dtype, T, experts, top, hidden
         close(got, want, dtype, "the sum")
 
 
+@pytest.mark.parametrize("rows, width, out", [(3, 64, 40), (17, 64, 40), (65, 96, 50), (700, 256, 1000)])
+def test_a_bias_that_bfloat16_holds_goes_into_the_library_s_product(rows, width, out):
+    x, weight = rand(rows, width, seed=1).to(torch.bfloat16), (rand(out, width, seed=2) / width ** 0.5).to(torch.bfloat16)
+    bias = rand(out, seed=3).to(torch.bfloat16).float()
+    want = (x.float() @ weight.float().T + bias).to(torch.bfloat16)
+    got = ops().linear(x.to(DEV), weight.to(DEV), bias.to(DEV), bias16=bias.to(torch.bfloat16).to(DEV))
+    close(got.float(), want.float(), torch.bfloat16, "with the bias in the product")
+    apart = ops().linear(x.to(DEV), weight.to(DEV), bias.to(DEV))
+    assert float((got.float() - apart.float()).abs().max()) <= 2.0 ** -7 * float(want.abs().max()), "one rounding either way"
+    from macllm_infer_amd.parts import BuildContext, Linear
+    build = BuildContext(hidden_size=width, dtype=torch.bfloat16, device=torch.device(DEV), max_context=64)
+    assert Linear([weight], [bias], build).bias16 is not None and Linear([weight], [bias + 1e-4], build).bias16 is None
+
+
 # ------------------------------------------------------------------ every mechanism alone
 def mixer_parts(layer, hidden, seed, sharpen=1.0):
     """(spec, tensors under the part's names, the design's mixer table, tensors under the stored names)."""
