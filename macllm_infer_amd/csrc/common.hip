@@ -27,31 +27,55 @@ extern "C" int mi_embed(const int* ids, const void* table, int table_dtype, floa
 }
 
 // The same through an RMS norm on the way into the stream: e = table[ids[t], :] * multiplier,
-// h[t, :] = e / sqrt(mean(e^2) + eps) * weight.  One workgroup a token; the row is read twice, the second time from a cache.
-template <typename T>
-__global__ void __launch_bounds__(256)
+// h[t, :] = e / sqrt(mean(e^2) + eps) * weight.  One workgroup a token; a thread keeps PER elements of the row in registers.
+template <typename T, int PER>
+__global__ void __launch_bounds__(1024)
 embed_rmsnorm_kernel(const int* __restrict__ ids, const T* __restrict__ table, float multiplier,
                      const float* __restrict__ weight, float eps, float* __restrict__ h, int d) {
   __shared__ float scratch[16];
   const long token = blockIdx.x;
   const T* row = table + (long)ids[token] * d;
   float* out = h + token * d;
+  float e[PER], w[PER];
   float squares = 0.f;
-  for (int i = threadIdx.x; i < d; i += blockDim.x) {
-    const float e = to_float(row[i]) * multiplier;
-    squares = fmaf(e, e, squares);
+#pragma unroll
+  for (int k = 0; k < PER; ++k) {
+    const int i = threadIdx.x + k * blockDim.x;
+    w[k] = i < d ? weight[i] : 0.f;
+    e[k] = i < d ? to_float(row[i]) * multiplier : 0.f;
   }
+#pragma unroll
+  for (int k = 0; k < PER; ++k) squares = fmaf(e[k], e[k], squares);
   const float rms = sqrtf(block_sum(squares, scratch) / (float)d + eps);
-  for (int i = threadIdx.x; i < d; i += blockDim.x) out[i] = to_float(row[i]) * multiplier / rms * weight[i];
+#pragma unroll
+  for (int k = 0; k < PER; ++k) {
+    const int i = threadIdx.x + k * blockDim.x;
+    if (i < d) out[i] = e[k] / rms * w[k];
+  }
+}
+
+template <typename T>
+static void launch_embed_rmsnorm(const int* ids, const T* table, float multiplier, const float* weight, float eps, float* h,
+                                 int tokens, int d, hipStream_t stream) {
+  // few tokens: as many threads as a row has elements, as far as they go; many tokens: smaller workgroups
+  const int most = tokens <= 512 ? 1024 : 256;
+  int per = 1;
+  while (per < 16 && (d + per - 1) / per > most) per *= 2;
+  const int threads = (((d + per - 1) / per + WAVE - 1) / WAVE) * WAVE;
+#define EMBED_CASE(PER_) \
+  if (per == PER_) embed_rmsnorm_kernel<T, PER_><<<tokens, threads, 0, stream>>>(ids, table, multiplier, weight, eps, h, d);
+  EMBED_CASE(1) EMBED_CASE(2) EMBED_CASE(4) EMBED_CASE(8) EMBED_CASE(16)
+#undef EMBED_CASE
 }
 
 extern "C" int mi_embed_rmsnorm(const int* ids, const void* table, int table_dtype, float multiplier, const float* weight,
                                 float eps, float* h, int T, int d, hipStream_t stream) {
   if (!ids || !table || !weight || !h || T <= 0 || d <= 0) return ERR_BAD_ARGUMENT;
+  if (d > 16384) return ERR_UNSUPPORTED_SIZE;
   if (table_dtype == DT_F32)
-    embed_rmsnorm_kernel<float><<<T, 256, 0, stream>>>(ids, (const float*)table, multiplier, weight, eps, h, d);
+    launch_embed_rmsnorm<float>(ids, (const float*)table, multiplier, weight, eps, h, T, d, stream);
   else if (table_dtype == DT_BF16)
-    embed_rmsnorm_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, (const bf16_t*)table, multiplier, weight, eps, h, d);
+    launch_embed_rmsnorm<bf16_t>(ids, (const bf16_t*)table, multiplier, weight, eps, h, T, d, stream);
   else
     return ERR_BAD_ARGUMENT;
   RETURN_IF_LAUNCH_FAILED();

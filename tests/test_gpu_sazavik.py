@@ -61,7 +61,7 @@ def test_branches_join_the_stream_through_an_rms_norm_of_their_own(out_dtype, d,
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T, d", [(1, 48), (33, 250), (300, 1024), (2, 5000)])
+@pytest.mark.parametrize("T, d", [(1, 48), (33, 250), (300, 1024), (700, 1030), (2, 3000), (2, 5000), (3, 16384)])
 def test_the_embedding_through_a_norm(dtype, T, d):
     table = rand(50, d, seed=1, scale=3.0).to(dtype)
     ids = torch.randint(0, 50, (T,), generator=torch.Generator().manual_seed(2)).to(torch.int32)
