@@ -121,7 +121,9 @@ class Engine:
             raise ConfigError("config.json: " + "; ".join(limit.text(self.spec.field_names) for limit in beyond))
         source = WeightSource.from_dir(model_dir) if model_dir is not None else WeightSource.from_tensors(tensors)
         if check_device:
-            kernel_build.ensure_modules(DecoderModel.kernel_modules(self.spec) + list(kernel_build.HOST_MODULES))
+            # (bfloat16 products of few rows go through the skinny kernels)
+            skinny = ["decode"] if self.dtype == torch.bfloat16 else []
+            kernel_build.ensure_modules(DecoderModel.kernel_modules(self.spec) + skinny + list(kernel_build.HOST_MODULES))
         source.apply_aliases(self.spec.tensor_aliases, root_prefix=self.spec.root_namespace)
         expected = DecoderModel.expected_tensors(self.spec)
         if self.spec.stored_name_rules:

@@ -44,6 +44,14 @@ class Attention(Mixer):
     query_tile = 64          # tokens of one lane that a workgroup of the prompt attention kernels takes
 
     @classmethod
+    def modules_of(cls, spec) -> tuple:
+        own_width = spec.head_dim in (64, 128) and spec.value_width == spec.head_dim
+        unused = {"mamba2"} if spec.conv_kernel == 0 else set()                  # the convolutions' kernels
+        if own_width or spec.head_dim % 8 or spec.head_dim > 128:                # the prompt kernel at padded widths
+            unused.add("attention_widths")
+        return tuple(name for name in cls.kernel_modules if name not in unused)
+
+    @classmethod
     def expected_tensors(cls, spec, prefix: str, hidden_size: int):
         q_rows = spec.num_heads * spec.head_dim
         kv_rows = spec.num_kv_heads * spec.head_dim

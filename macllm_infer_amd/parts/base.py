@@ -194,6 +194,11 @@ class Part:
     graph_safe = False
 
     @classmethod
+    def modules_of(cls, spec) -> tuple:
+        """The HIP modules that a part of this spec launches: all of the class's, unless some are for forms it has not."""
+        return tuple(cls.kernel_modules)
+
+    @classmethod
     def expected_tensors(cls, spec, prefix: str, hidden_size: int):
         return []
 

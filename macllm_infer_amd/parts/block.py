@@ -113,7 +113,8 @@ class ParallelPreNormBlock:
     def kernel_modules(cls, layer):
         modules = []
         for spec in cls._part_specs(layer):
-            modules += list(part_class(spec).kernel_modules)
+            part = part_class(spec)
+            modules += list(part.modules_of(spec) if hasattr(part, "modules_of") else part.kernel_modules)
         return modules
 
     def __init__(self, layer, tensors, build: BuildContext):
