@@ -316,10 +316,10 @@ def plain_mixer(kind, x, table, stored, eps=1e-5):
 LAYERS = [
     sazavik_configs.chunked(6, 2, 8, 12, 21, 4, base=300.0), sazavik_configs.chunked(4, 1, 64, 64, 40, 64),
     sazavik_configs.chunked(3, 3, 128, 128, 64, 32, base=1e6), sazavik_configs.chunked(5, 1, 24, 40, 5, 24),
-    sazavik_configs.chunked(2, 2, 96, 96, 300, 24), sazavik_configs.chunked(4, 2, 16, 16, None, 8),
-    sazavik_configs.chunked(4, 2, 20, 12, 33, 20, halves=True), sazavik_configs.chunked(8, 2, 64, 64, 100, 32, halves=True),
+    sazavik_configs.chunked(2, 2, 96, 96, 300, 40), sazavik_configs.chunked(4, 2, 16, 16, None, 8),
+    sazavik_configs.chunked(4, 2, 20, 12, 33, 20, halves=True), sazavik_configs.chunked(6, 2, 64, 64, 100, 48, halves=True),
     sazavik_configs.chunked(1, 1, 48, 128, 16, 48, halves=True, scale=0.3), sazavik_configs.chunked(2, 1, 128, 128, 1, 128, halves=True),
-    sazavik_configs.distant(3, 1, 10, 6, 13, every=7), sazavik_configs.distant(8, 8, 48, 48, 60, coef=0.5, every=32),
+    sazavik_configs.distant(3, 1, 10, 6, 13, every=7), sazavik_configs.distant(7, 7, 48, 40, 60, coef=0.6, every=32),
     sazavik_configs.distant(6, 2, 64, 64, 37, every=64), sazavik_configs.distant(5, 5, 7, 9, 11, coef=-0.2, every=3),
     sazavik_configs.distant(12, 2, 128, 128, 90, every=1), sazavik_configs.distant(4, 1, 32, 256, None, every=None),
 ]
